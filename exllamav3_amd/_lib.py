@@ -236,7 +236,7 @@ def _declare(l):
 # ---- the sequence-mixer library (include/exl3_mix.h, csrc/mix_*.hip) -------------------------------------------------------------
 MIX_LIB_PATH = os.path.join(_HERE, "libexl3_mix.so")
 MIX_HEADER_PATH = os.path.join(os.path.dirname(_HERE), "include", "exl3_mix.h")
-MIX_ABI_VERSION = 4
+MIX_ABI_VERSION = 5
 _mix = None
 
 
@@ -319,17 +319,19 @@ def _declare_mix(l):
     sig("exl3_mix_act", vp, vp, i64, i32, i32, i32, i32, vp)
     sig("exl3_mix_glu_act", vp, vp, i64, vp, i64, i32, i32, i32, f32, i32, vp)
     sig("exl3_mix_token_gate", vp, vp, i64, vp, i64, i32, vp, i32, i32, i32, i32, vp)
-    sig("exl3_mix_heads_gate", vp, vp, i64, i64, vp, i64, i32, i32, i32, i32, vp)
+    sig("exl3_mix_heads_gate", vp, i64, vp, i64, i64, vp, i64, i32, i32, i32, i32, vp)
     sig("exl3_mix_topk_sigmoid", vp, vp, vp, vp, f32, i32, i32, i32, i32, vp)
     sig("exl3_mix_latent_prep", vp, vp, vp, i64, vp, vp, i64, vp, vp, vp, vp, vp, f32, f32, i32, i32, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_latent_fill_k", vp, i64, vp, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_latent_decode_mfma_scratch", i32, i32, i32, i32, ctypes.POINTER(i64))
-    sig("exl3_mix_latent_decode_mfma", vp, i64, i64, vp, i64, i64, vp, i64, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, i32, vp)
-    sig("exl3_mix_latent_decode", vp, i64, i64, vp, i64, i64, vp, i64, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, i32, vp)
-    sig("exl3_mix_attn_prefill_ex", vp, i32, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, vp)
-    sig("exl3_mix_attn_prefill_mfma_ex", vp, i32, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, i32, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, vp)
-    sig("exl3_mix_attn_decode_ex", vp, i32, vp, i64, vp, vp, vp, i64, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, vp)
-    sig("exl3_mix_qk_prep", vp, i64, vp, i64, vp, i64, vp, vp, vp, i32, f32, i32, f32, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_latent_decode_mfma", vp, i64, i64, vp, i64, i64, vp, i64, vp, vp, vp, vp, vp, i64, i32, vp, i32, i32, i32, i32, i32, i32, f32, i32, vp)
+    sig("exl3_mix_latent_rows", vp, vp, vp, i64, vp, vp, vp, i64, vp, i32, vp, i64, i32, vp, vp, vp, vp, f32, i32, f32, i32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_rotate_heads", vp, i64, vp, vp, f32, i32, i32, i32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_latent_decode", vp, i64, i64, vp, i64, i64, vp, i64, vp, vp, vp, vp, vp, i64, i32, i32, i32, i32, i32, i32, f32, i32, i32, vp)
+    sig("exl3_mix_attn_prefill_ex", vp, i64, i32, vp, i64, vp, i64, vp, i64, vp, i64, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_attn_prefill_mfma_ex", vp, i64, i32, vp, i64, vp, i64, vp, i64, vp, i64, i32, vp, vp, i32, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, vp)
+    sig("exl3_mix_attn_decode_ex", vp, i64, i32, vp, i64, vp, vp, vp, i64, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, vp)
+    sig("exl3_mix_qk_prep", vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, i32, f32, i32, f32, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_diff_combine", vp, vp, f32, f32, f32, vp, i64, i32, i32, i32, i32, vp)
     sig("exl3_mix_residual_rms", vp, vp, i64, i32, vp, f32, vp, i64, vp, i32, vp, vp, vp, vp, i32, i32, i32, vp)
     sig("exl3_mix_canon", vp, i64, vp, i64, vp, i32, vp, vp, vp, vp, vp, vp, i32, i32, i32, vp)
@@ -343,7 +345,8 @@ def _declare_mix(l):
     sig("exl3_mix_embed_sinusoid", vp, vp, vp, vp, vp, f32, i32, i32, i32, i32, vp)
     sig("exl3_mix_layer_norm_rows", vp, vp, vp, vp, vp, f32, i32, i32, i32, vp)
     sig("exl3_mix_residual_norm_conv", vp, vp, i64, vp, i64, f32, i32, i32, vp, vp, f32, vp, i64, vp, i64, vp, i32, vp, vp, vp, vp, i32, i32, i32, vp)
-    sig("exl3_mix_glu_act_rowgate", vp, vp, i64, vp, i64, vp, i64, i32, i32, i32, f32, i32, vp)
+    sig("exl3_mix_residual_norm_pair", vp, vp, i64, i32, vp, vp, i64, vp, vp, i64, f32, i32, i32, i32, vp)
+    sig("exl3_mix_glu_act_rowgate", vp, i64, vp, i64, vp, i64, vp, i64, i32, i32, i32, f32, i32, vp)
     sig("exl3_mix_topk_grouped_ex", vp, vp, vp, vp, vp, i32, f32, i32, i32, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_paged_store", vp, vp, vp, i64, vp, i64, vp, i64, i32, vp, vp, vp, i32, i32, i32, i32, vp)
     sig("exl3_mix_sigattn_prefill", vp, vp, i64, vp, i64, vp, i64, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, vp)
@@ -352,5 +355,7 @@ def _declare_mix(l):
     sig("exl3_mix_mlstm_scan", vp, vp, vp, vp, vp, i64, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, vp, i32, i32, i32, i32, f32, f32, i32, vp)
     sig("exl3_mix_delta_prep", vp, vp, vp, vp, vp, vp, i64, vp, i32, vp, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, vp)
     sig("exl3_mix_delta_scan", vp, vp, vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp)
-    sig("exl3_mix_head_norm_gate", vp, vp, vp, i32, vp, i64, i32, f32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_retention", vp, vp, vp, i64, vp, i64, vp, i64, vp, i32, vp, i32, i32, vp, vp, vp, i32, i32, i32, i32, f32, i32, i32, vp, i32, vp)
+    sig("exl3_mix_retention_step", vp, i64, vp, vp, i64, vp, i64, vp, i64, vp, i64, vp, i32, vp, i32, i32, vp, vp, i32, i32, i32, i32, f32, f32, i32, vp)
+    sig("exl3_mix_head_norm_gate", vp, i64, vp, vp, i32, vp, i64, i32, f32, i32, i32, i32, i32, vp)
     sig("exl3_mix_rms_pair", vp, vp, i64, vp, vp, i64, vp, f32, f32, i32, i32, i32, vp)

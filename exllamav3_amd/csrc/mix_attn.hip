@@ -38,12 +38,13 @@ __global__ __launch_bounds__(64) void attn_store_kernel(T* __restrict__ v_norm, 
 
 // `maps` attention maps per head (differential attention: 2): queries are laid out [head][map][dim], keys [kv head][map][dim], every map of a head reads
 // the values of the head's key/value head, and the result is [row][head][map][vdim].  mask 0: the last `window` positions; 1: the positions of the row's
-// own chunk of `window` positions (a chunk starts where the position is a multiple of `window`).
+// own chunk of `window` positions (a chunk starts where the position is a multiple of `window`).  keep: the first `keep` positions stay visible whatever the mask
+// says.  gate: one number per head (gate_cols 1) or one per value element (gate_cols vdim).
 template <typename T, int MAXV, typename TO, int NW>
-__global__ __launch_bounds__(64 * NW) void attn_prefill_kernel(TO* __restrict__ out, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ k, int64_t k_ld,
-                                                          const T* __restrict__ v, int64_t v_ld, const T* __restrict__ gate, int64_t gate_ld, const float* __restrict__ sink,
+__global__ __launch_bounds__(64 * NW) void attn_prefill_kernel(TO* __restrict__ out, int64_t out_ld, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ k, int64_t k_ld,
+                                                          const T* __restrict__ v, int64_t v_ld, const T* __restrict__ gate, int64_t gate_ld, int gate_cols, const float* __restrict__ sink,
                                                           const int32_t* __restrict__ cu, const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
-                                                          int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask)
+                                                          int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep)
 {
     extern __shared__ float smem[];
     const int n = blockIdx.x, h = blockIdx.y;                 // h counts (head, map)
@@ -51,18 +52,29 @@ __global__ __launch_bounds__(64 * NW) void attn_prefill_kernel(TO* __restrict__ 
     const int b = tok_seq[n], first = cu[b];
     const int i = n - first;                                  // the row's place in its sequence == its position (the sequence starts in this step)
     const int lo = mask == EXL3_MIX_MASK_CHUNK ? (i / window) * window : max(0, i - window + 1);
-    const float gt = gate ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) : 1.0f;
+    const bool by_head = gate && gate_cols == 1;
+    const float gt = by_head ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) : 1.0f;
+    const T* grow = gate && !by_head ? gate + (int64_t) n * gate_ld + (int64_t) h * vdim : nullptr;
+    if (keep > 0)                                             // keys 0 .. keep - 1, then lo .. i
+    {
+        const int kept = min(keep, lo);
+        const T* k0 = k + (int64_t) first * k_ld + (int64_t) kh * dim;
+        attn_row<T, MAXV, TO, NW, row_jump>(out + (int64_t) n * out_ld + (int64_t) h * vdim, q + (int64_t) n * q_ld + (int64_t) h * dim, q, dim, k0, k_ld,
+                              v + (int64_t) first * v_ld + (int64_t) g * vdim, v_ld, kept + i - lo + 1, dim, vdim, scale, sink != nullptr, sink ? sink[h] : 0.f, gt,
+                              rows_are_16_byte(k0, k_ld, dim), smem, softcap, row_jump{kept, (int64_t) (lo - kept)}, grow);
+        return;
+    }
     const T* kb = k + (int64_t) (first + lo) * k_ld + (int64_t) kh * dim;
-    attn_row<T, MAXV, TO, NW>(out + ((int64_t) n * heads * maps + h) * vdim, q + (int64_t) n * q_ld + (int64_t) h * dim, q, dim, kb, k_ld,
+    attn_row<T, MAXV, TO, NW>(out + (int64_t) n * out_ld + (int64_t) h * vdim, q + (int64_t) n * q_ld + (int64_t) h * dim, q, dim, kb, k_ld,
                           v + (int64_t) (first + lo) * v_ld + (int64_t) g * vdim, v_ld,
-                          i - lo + 1, dim, vdim, scale, sink != nullptr, sink ? sink[h] : 0.f, gt, rows_are_16_byte(kb, k_ld, dim), smem, softcap);
+                          i - lo + 1, dim, vdim, scale, sink != nullptr, sink ? sink[h] : 0.f, gt, rows_are_16_byte(kb, k_ld, dim), smem, softcap, row_linear(), grow);
 }
 
 // Rings: ring_k [slots][window][kv_heads * maps][dim], ring_v [slots][window][kv_heads][vdim], entry = position % window.  mask 0: the newest
 // min(len, window) entries (all of them, in any order); 1: the row's chunk, which is the entries 0 .. (len - 1) % window.
 template <typename T, int MAXV, typename TO, int NW>
-__global__ __launch_bounds__(64 * NW) void attn_decode_kernel(TO* __restrict__ out, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ ring_k,
-                                                         const T* __restrict__ ring_v, const T* __restrict__ gate, int64_t gate_ld, const float* __restrict__ sink,
+__global__ __launch_bounds__(64 * NW) void attn_decode_kernel(TO* __restrict__ out, int64_t out_ld, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ ring_k,
+                                                         const T* __restrict__ ring_v, const T* __restrict__ gate, int64_t gate_ld, int gate_cols, const float* __restrict__ sink,
                                                          const int32_t* __restrict__ slots, const int32_t* __restrict__ len_after,
                                                          int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask)
 {
@@ -72,11 +84,13 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_kernel(TO* __restrict__ o
     const int len = len_after[n];
     const int count = mask == EXL3_MIX_MASK_CHUNK ? (len - 1) % window + 1 : min(len, window);
     const int64_t row0 = (int64_t) slots[n] * window;
-    const float gt = gate ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) : 1.0f;
+    const bool by_head = gate && gate_cols == 1;
+    const float gt = by_head ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) : 1.0f;
+    const T* grow = gate && !by_head ? gate + (int64_t) n * gate_ld + (int64_t) h * vdim : nullptr;
     const T* kb = ring_k + (row0 * kheads + kh) * dim;
-    attn_row<T, MAXV, TO, NW>(out + ((int64_t) n * heads * maps + h) * vdim, q + (int64_t) n * q_ld + (int64_t) h * dim, q, dim,
+    attn_row<T, MAXV, TO, NW>(out + (int64_t) n * out_ld + (int64_t) h * vdim, q + (int64_t) n * q_ld + (int64_t) h * dim, q, dim,
                           kb, (int64_t) kheads * dim, ring_v + (row0 * kv_heads + g) * vdim, (int64_t) kv_heads * vdim,
-                          count, dim, vdim, scale, sink != nullptr, sink ? sink[h] : 0.f, gt, rows_are_16_byte(kb, (int64_t) kheads * dim, dim), smem, softcap);
+                          count, dim, vdim, scale, sink != nullptr, sink ? sink[h] : 0.f, gt, rows_are_16_byte(kb, (int64_t) kheads * dim, dim), smem, softcap, row_linear(), grow);
 }
 
 extern "C" int exl3_mix_attn_store(void* v_norm, void* ring_k, void* ring_v, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
@@ -111,8 +125,11 @@ extern "C" int exl3_mix_attn_store(void* v_norm, void* ring_k, void* ring_v, con
         MIX_DISPATCH_T(dtype, if (out_f32) ATTN_LAUNCH_TO(KERNEL, float, __VA_ARGS__); else ATTN_LAUNCH_TO(KERNEL, T, __VA_ARGS__)); \
     } while (0)
 
-static int attn_check(const char* what, int n, int heads, int kv_heads, int maps, int dim, int vdim, int window, int mask, float softcap, const void* gate)
+static int attn_check(const char* what, int n, int heads, int kv_heads, int maps, int dim, int vdim, int window, int mask, float softcap, const void* gate, int gate_cols,
+                      int64_t gate_ld, int64_t out_ld)
 {
+    MIX_CHECK(out_ld >= (int64_t) heads * maps * vdim && (!gate || ((gate_cols == 1 || gate_cols == vdim) && gate_ld >= (int64_t) heads * gate_cols)),
+              "%s: bad row stride of the result or the gate (a gate has 1 or vdim columns per head)", what);
     MIX_CHECK(n >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "%s: heads %d must be a multiple of kv_heads %d", what, heads, kv_heads);
     MIX_CHECK(maps >= 1 && heads * maps <= 65535 && (maps == 1 || !gate), "%s: %d maps per head (a gate per head applies to one map only)", what, maps);
     MIX_CHECK((mask == EXL3_MIX_MASK_WINDOW || mask == EXL3_MIX_MASK_CHUNK) && softcap >= 0.f, "%s: unknown mask %d or a negative softcap", what, mask);
@@ -120,18 +137,19 @@ static int attn_check(const char* what, int n, int heads, int kv_heads, int maps
     return EXL3_MIX_OK;
 }
 
-extern "C" int exl3_mix_attn_prefill_ex(void* out, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
-                                        const void* gate, int64_t gate_ld, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
-                                        int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int dtype, void* stream)
+extern "C" int exl3_mix_attn_prefill_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
+                                        const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
+                                        int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, int dtype, void* stream)
 {
     MIX_CHECK(out && q && k && v && cu && tok_seq && tok_pos, "mix_attn_prefill: null pointer");
-    if (int rc = attn_check("mix_attn_prefill", n, heads, kv_heads, maps, dim, vdim, window, mask, softcap, gate)) return rc;
-    MIX_CHECK(q_ld >= (int64_t) heads * maps * dim && k_ld >= (int64_t) kv_heads * maps * dim && v_ld >= (int64_t) kv_heads * vdim && (!gate || gate_ld >= heads),
+    if (int rc = attn_check("mix_attn_prefill", n, heads, kv_heads, maps, dim, vdim, window, mask, softcap, gate, gate_cols, gate_ld, out_ld)) return rc;
+    MIX_CHECK(q_ld >= (int64_t) heads * maps * dim && k_ld >= (int64_t) kv_heads * maps * dim && v_ld >= (int64_t) kv_heads * vdim,
               "mix_attn_prefill: bad row strides");
+    MIX_CHECK(keep >= 0 && (keep == 0 || mask == EXL3_MIX_MASK_WINDOW), "mix_attn_prefill: kept first tokens go with a window");
     if (n == 0) return EXL3_MIX_OK;
     const bool wide = false;
-    ATTN_LAUNCH(attn_prefill_kernel, (const T*) q, q_ld, (const T*) k, k_ld, (const T*) v, v_ld, (const T*) gate, gate_ld, sink, cu, tok_seq, tok_pos,
-                heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask);
+    ATTN_LAUNCH(attn_prefill_kernel, out_ld, (const T*) q, q_ld, (const T*) k, k_ld, (const T*) v, v_ld, (const T*) gate, gate_ld, gate_cols, sink, cu, tok_seq, tok_pos,
+                heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep);
     return mix_check_launch("mix_attn_prefill");
 }
 
@@ -139,20 +157,20 @@ extern "C" int exl3_mix_attn_prefill(void* out, const void* q, int64_t q_ld, con
                                      const void* gate, int64_t gate_ld, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
                                      int n, int heads, int kv_heads, int dim, int vdim, float scale, int window, int dtype, void* stream)
 {
-    return exl3_mix_attn_prefill_ex(out, 0, q, q_ld, k, k_ld, v_norm, (int64_t) kv_heads * vdim, gate, gate_ld, sink, cu, tok_seq, tok_pos, n, heads, kv_heads, 1, dim, vdim,
-                                    scale, 0.f, window, EXL3_MIX_MASK_WINDOW, dtype, stream);
+    return exl3_mix_attn_prefill_ex(out, (int64_t) heads * vdim, 0, q, q_ld, k, k_ld, v_norm, (int64_t) kv_heads * vdim, gate, gate_ld, 1, sink, cu, tok_seq, tok_pos, n, heads, kv_heads, 1, dim, vdim,
+                                    scale, 0.f, window, EXL3_MIX_MASK_WINDOW, 0, dtype, stream);
 }
 
-extern "C" int exl3_mix_attn_decode_ex(void* out, int out_f32, const void* q, int64_t q_ld, const void* ring_k, const void* ring_v,
-                                       const void* gate, int64_t gate_ld, const float* sink, const int32_t* slots, const int32_t* len_after,
+extern "C" int exl3_mix_attn_decode_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* ring_k, const void* ring_v,
+                                       const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* slots, const int32_t* len_after,
                                        int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int dtype, void* stream)
 {
     MIX_CHECK(out && q && ring_k && ring_v && slots && len_after, "mix_attn_decode: null pointer");
-    if (int rc = attn_check("mix_attn_decode", n, heads, kv_heads, maps, dim, vdim, window, mask, softcap, gate)) return rc;
-    MIX_CHECK(q_ld >= (int64_t) heads * maps * dim && (!gate || gate_ld >= heads), "mix_attn_decode: bad row strides");
+    if (int rc = attn_check("mix_attn_decode", n, heads, kv_heads, maps, dim, vdim, window, mask, softcap, gate, gate_cols, gate_ld, out_ld)) return rc;
+    MIX_CHECK(q_ld >= (int64_t) heads * maps * dim, "mix_attn_decode: bad row strides");
     if (n == 0) return EXL3_MIX_OK;
     const bool wide = (int64_t) n * heads * maps <= 256 && window > 256 && vdim <= 256;
-    ATTN_LAUNCH(attn_decode_kernel, (const T*) q, q_ld, (const T*) ring_k, (const T*) ring_v, (const T*) gate, gate_ld, sink, slots, len_after,
+    ATTN_LAUNCH(attn_decode_kernel, out_ld, (const T*) q, q_ld, (const T*) ring_k, (const T*) ring_v, (const T*) gate, gate_ld, gate_cols, sink, slots, len_after,
                 heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask);
     return mix_check_launch("mix_attn_decode");
 }
@@ -161,6 +179,6 @@ extern "C" int exl3_mix_attn_decode(void* out, const void* q, int64_t q_ld, cons
                                     const void* gate, int64_t gate_ld, const float* sink, const int32_t* slots, const int32_t* len_after,
                                     int n, int heads, int kv_heads, int dim, int vdim, float scale, int window, int dtype, void* stream)
 {
-    return exl3_mix_attn_decode_ex(out, 0, q, q_ld, ring_k, ring_v, gate, gate_ld, sink, slots, len_after, n, heads, kv_heads, 1, dim, vdim, scale, 0.f, window,
+    return exl3_mix_attn_decode_ex(out, (int64_t) heads * vdim, 0, q, q_ld, ring_k, ring_v, gate, gate_ld, 1, sink, slots, len_after, n, heads, kv_heads, 1, dim, vdim, scale, 0.f, window,
                                    EXL3_MIX_MASK_WINDOW, dtype, stream);
 }

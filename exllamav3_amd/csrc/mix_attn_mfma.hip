@@ -17,7 +17,8 @@
 // head's key/value head; result [row][head][map][vdim]); a chunk mask (a row sees the positions of its own chunk of `window` positions) beside the
 // sliding window -- both give every row a first visible key lo(i) that never decreases with i, which is all the tile logic uses; a soft cap on the
 // scores, cap tanh(score / cap), applied to the scaled scores before the running maximum (tanh is increasing, so the largest raw score still is the
-// largest score); and a float32 result.
+// largest score); a float32 result; the first `keep` positions visible to every row beside its window (the tiles that hold them are visited first, then
+// those of the window: a row's mask is "in the window, or among the first"); and an output gate per head or per value element, applied in the epilogue.
 #include "mix_common.cuh"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -33,11 +34,11 @@ typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ int first_visible(int i, int window, int mask) { return mask == EXL3_MIX_MASK_CHUNK ? (i / window) * window : i - window + 1; }
 
 template <int KD, int NV, int AM_KEYS, bool CAP>
-__global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __restrict__ out_any, int out_f32, const bf16_t* __restrict__ q, int64_t q_ld, const bf16_t* __restrict__ k,
-                                                                int64_t k_ld, const bf16_t* __restrict__ v_norm, int64_t v_ld, const bf16_t* __restrict__ gate, int64_t gate_ld,
+__global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __restrict__ out_any, int64_t out_ld, int out_f32, const bf16_t* __restrict__ q, int64_t q_ld, const bf16_t* __restrict__ k,
+                                                                int64_t k_ld, const bf16_t* __restrict__ v_norm, int64_t v_ld, const bf16_t* __restrict__ gate, int64_t gate_ld, int gate_cols,
                                                                 const float* __restrict__ sink, const int32_t* __restrict__ cu,
-                                                                int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask,
-                                                                int k_vec, int v_vec)
+                                                                int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep,
+                                                                int k_vec, int v_vec, int o_vec)
 {
     constexpr int DP = KD * 32, KS = DP + AM_PAD, VS = AM_KEYS + AM_PAD;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
@@ -46,7 +47,7 @@ __global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __r
 
     const int b = blockIdx.y, h = blockIdx.z;
     const int first = cu[b], len = cu[b + 1] - first;
-    const int q0 = blockIdx.x * AM_ROWS;
+    const int q0 = (gridDim.x - 1 - blockIdx.x) * AM_ROWS;        // the blocks with the most keys start first
     if (q0 >= len) return;
     const int hh = h / maps;                                      // h counts (head, map)
     const int vh = hh / (heads / kv_heads), kvh = vh * maps + (h - hh * maps);
@@ -82,7 +83,8 @@ __global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __r
     const int j_begin = (max(0, first_visible(q0, window, mask)) / AM_KEYS) * AM_KEYS;
     const int wave_lo = first_visible(wq_lo, window, mask), wave_hi_lo = first_visible(wq_hi, window, mask);      // first visible key of the wave's first / last row
     const int my_lo = first_visible(qi, window, mask);
-    for (int j0 = j_begin; j0 <= blk_hi; j0 += AM_KEYS)
+    const int keep_end = keep > 0 ? min(j_begin, (keep + AM_KEYS - 1) / AM_KEYS * AM_KEYS) : 0;        // the kept first positions' tiles ahead of the window's
+    for (int j0 = keep_end > 0 ? 0 : j_begin; j0 <= blk_hi; j0 = (j0 + AM_KEYS == keep_end) ? j_begin : j0 + AM_KEYS)
     {
         __syncthreads();                                           // the previous tile's operand reads are over
         // stage K [32][DP] (zero beyond dim / len) and V^T [vdim][32]
@@ -117,7 +119,7 @@ __global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __r
         }
         __syncthreads();
         // tiles wholly outside this wave's windows: nothing to add (uniform per wave; the barriers above are still met)
-        const bool skip = !wave_live || j0 > wq_hi || j0 + AM_KEYS - 1 < wave_lo;
+        const bool skip = !wave_live || j0 > wq_hi || (j0 + AM_KEYS - 1 < wave_lo && j0 >= keep);
         if (!skip)
         {
             constexpr int NS = AM_KEYS / 16;                                   // 16-key score tiles
@@ -168,7 +170,7 @@ __global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __r
                     for (int i = 0; i < 4; ++i)
                     {
                         const int j = j0 + u * 16 + g * 4 + i;
-                        const bool ok = j <= qi && j >= my_lo && qi < len;
+                        const bool ok = j <= qi && (j >= my_lo || j < keep) && qi < len;
                         sc[u][i] = ok ? sc[u][i] : -INFINITY;
                         mx = fmaxf(mx, sc[u][i]);
                     }
@@ -217,20 +219,42 @@ __global__ __launch_bounds__(AM_THREADS) void attn_prefill_mfma_kernel(void* __r
     l += __shfl_xor(l, 32, 64);
     if (qi >= len) return;
     const int64_t n = first + qi;
-    const float gt = gate ? sigmoid_f(to_f(gate[n * gate_ld + h])) : 1.0f;
+    const bool by_head = gate && gate_cols == 1;
+    const float gt = by_head ? sigmoid_f(to_f(gate[n * gate_ld + h])) : 1.0f;
+    const bf16_t* grow = gate && !by_head ? gate + n * gate_ld + (int64_t) h * vdim : nullptr;
     const float f = (l > 0.f ? 1.0f / l : 0.f) * gt;
-    const int64_t o0 = (n * heads * maps + h) * vdim;
+    const int64_t o0 = n * out_ld + (int64_t) h * vdim;
     #pragma unroll
     for (int t = 0; t < NV; ++t)
     {
+        const int col0 = t * 16 + g * 4;                           // four neighbouring value columns per lane and tile
+        if (o_vec && col0 + 4 <= vdim)                             // bfloat16 result and gate rows in 8-byte groups (host-checked alignment)
+        {
+            float r[4];
+            #pragma unroll
+            for (int i = 0; i < 4; ++i) r[i] = acc[t][i] * f;
+            if (grow)
+            {
+                union { uint2 v; bf16_t e[4]; } gv;
+                gv.v = *(const uint2*) (grow + col0);
+                #pragma unroll
+                for (int i = 0; i < 4; ++i) r[i] *= sigmoid_f(to_f(gv.e[i]));
+            }
+            union { uint2 v; bf16_t e[4]; } ov;
+            #pragma unroll
+            for (int i = 0; i < 4; ++i) ov.e[i] = from_f<bf16_t>(r[i]);
+            *(uint2*) ((bf16_t*) out_any + o0 + col0) = ov.v;
+            continue;
+        }
         #pragma unroll
         for (int i = 0; i < 4; ++i)
         {
-            const int col = t * 16 + g * 4 + i;
+            const int col = col0 + i;
             if (col < vdim)
             {
-                if (out_f32) ((float*) out_any)[o0 + col] = acc[t][i] * f;
-                else         ((bf16_t*) out_any)[o0 + col] = from_f<bf16_t>(acc[t][i] * f);
+                const float r = acc[t][i] * f * (grow ? sigmoid_f(to_f(grow[col])) : 1.0f);
+                if (out_f32) ((float*) out_any)[o0 + col] = r;
+                else         ((bf16_t*) out_any)[o0 + col] = from_f<bf16_t>(r);
             }
         }
     }
@@ -240,13 +264,13 @@ extern "C" int exl3_mix_attn_prefill_mfma(void* out, const void* q, int64_t q_ld
                                           const void* gate, int64_t gate_ld, const float* sink, const int32_t* cu,
                                           int batch, int max_rows, int heads, int kv_heads, int dim, int vdim, float scale, int window, void* stream)
 {
-    return exl3_mix_attn_prefill_mfma_ex(out, 0, q, q_ld, k, k_ld, v_norm, (int64_t) kv_heads * vdim, gate, gate_ld, sink, cu, batch, max_rows, heads, kv_heads, 1, dim, vdim,
-                                         scale, 0.f, window, EXL3_MIX_MASK_WINDOW, stream);
+    return exl3_mix_attn_prefill_mfma_ex(out, (int64_t) heads * vdim, 0, q, q_ld, k, k_ld, v_norm, (int64_t) kv_heads * vdim, gate, gate_ld, 1, sink, cu, batch, max_rows, heads, kv_heads, 1, dim, vdim,
+                                         scale, 0.f, window, EXL3_MIX_MASK_WINDOW, 0, stream);
 }
 
-extern "C" int exl3_mix_attn_prefill_mfma_ex(void* out, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v_norm, int64_t v_ld,
-                                             const void* gate, int64_t gate_ld, const float* sink, const int32_t* cu,
-                                             int batch, int max_rows, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask,
+extern "C" int exl3_mix_attn_prefill_mfma_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v_norm, int64_t v_ld,
+                                             const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu,
+                                             int batch, int max_rows, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep,
                                              void* stream)
 {
     MIX_CHECK(out && q && k && v_norm && cu, "mix_attn_prefill_mfma: null pointer");
@@ -254,25 +278,29 @@ extern "C" int exl3_mix_attn_prefill_mfma_ex(void* out, int out_f32, const void*
               "mix_attn_prefill_mfma: heads %d / kv_heads %d / batch %d", heads, kv_heads, batch);
     MIX_CHECK((maps == 1 || !gate) && softcap >= 0.f && (mask == EXL3_MIX_MASK_WINDOW || mask == EXL3_MIX_MASK_CHUNK),
               "mix_attn_prefill_mfma: a gate per head applies to one map only; softcap >= 0; mask %d", mask);
+    MIX_CHECK(keep >= 0 && (keep == 0 || mask == EXL3_MIX_MASK_WINDOW), "mix_attn_prefill_mfma: kept first tokens go with a window");
     MIX_CHECK(dim > 0 && dim <= 256 && vdim > 0 && vdim <= 256 && window > 0, "mix_attn_prefill_mfma: dim %d and vdim %d must be <= 256", dim, vdim);
     MIX_CHECK(scale > 0.f, "mix_attn_prefill_mfma: the score scale must be positive (the running maximum is taken over raw scores)");
-    MIX_CHECK(q_ld >= (int64_t) heads * maps * dim && k_ld >= (int64_t) kv_heads * maps * dim && v_ld >= (int64_t) kv_heads * vdim && (!gate || gate_ld >= heads),
+    MIX_CHECK(q_ld >= (int64_t) heads * maps * dim && k_ld >= (int64_t) kv_heads * maps * dim && v_ld >= (int64_t) kv_heads * vdim && out_ld >= (int64_t) heads * maps * vdim &&
+              (!gate || ((gate_cols == 1 || gate_cols == vdim) && gate_ld >= (int64_t) heads * gate_cols)),
               "mix_attn_prefill_mfma: bad row strides");
     if (batch == 0 || max_rows == 0) return EXL3_MIX_OK;
     const dim3 grid((max_rows + AM_ROWS - 1) / AM_ROWS, batch, heads * maps);
     const int k_vec = ((uintptr_t) k % 16 == 0) && (k_ld % 8 == 0) && (dim % 8 == 0);
     const int v_vec = ((uintptr_t) v_norm % 16 == 0) && (v_ld % 8 == 0) && (vdim % 8 == 0);
+    const int o_vec = !out_f32 && vdim % 4 == 0 && out_ld % 4 == 0 && (uintptr_t) out % 8 == 0 && (!gate || gate_cols == 1 || (gate_ld % 4 == 0 && (uintptr_t) gate % 8 == 0));
     #define AM_LDS(KDV, NVV, KTV) ((size_t) (KTV * (KDV * 32 + AM_PAD) + NVV * 16 * (KTV + AM_PAD)) * sizeof(uint16_t))
     #define AM_LAUNCH_C(KDV, NVV, KTV, CAPV) \
-        hipLaunchKernelGGL((attn_prefill_mfma_kernel<KDV, NVV, KTV, CAPV>), grid, dim3(AM_THREADS), AM_LDS(KDV, NVV, KTV), (hipStream_t) stream, out, out_f32, (const bf16_t*) q, q_ld, \
-                           (const bf16_t*) k, k_ld, (const bf16_t*) v_norm, v_ld, (const bf16_t*) gate, gate_ld, sink, cu, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, \
-                           k_vec, v_vec)
+        hipLaunchKernelGGL((attn_prefill_mfma_kernel<KDV, NVV, KTV, CAPV>), grid, dim3(AM_THREADS), AM_LDS(KDV, NVV, KTV), (hipStream_t) stream, out, out_ld, out_f32, (const bf16_t*) q, q_ld, \
+                           (const bf16_t*) k, k_ld, (const bf16_t*) v_norm, v_ld, (const bf16_t*) gate, gate_ld, gate_cols, sink, cu, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, \
+                           k_vec, v_vec, o_vec)
     #define AM_LAUNCH(KDV, NVV, KTV) do { \
         static_assert(AM_LDS(KDV, NVV, KTV) <= 65536, "tile does not fit the LDS"); \
         if (softcap > 0.f) AM_LAUNCH_C(KDV, NVV, KTV, true); else AM_LAUNCH_C(KDV, NVV, KTV, false); } while (0)
     const int kd = (dim + 31) / 32, nv = (vdim + 15) / 16;
     if (kd <= 2)      { if (nv <= 4) AM_LAUNCH(2, 4, 64); else if (nv <= 8) AM_LAUNCH(2, 8, 64); else AM_LAUNCH(2, 16, 64); }
     else if (kd <= 4) { if (nv <= 4) AM_LAUNCH(4, 4, 64); else if (nv <= 8) AM_LAUNCH(4, 8, 64); else AM_LAUNCH(4, 16, 64); }
+    else if (kd <= 6) { if (nv <= 4) AM_LAUNCH(6, 4, 64); else if (nv <= 8) AM_LAUNCH(6, 8, 64); else AM_LAUNCH(6, 16, 64); }
     else              { if (nv <= 4) AM_LAUNCH(8, 4, 64); else if (nv <= 8) AM_LAUNCH(8, 8, 64); else AM_LAUNCH(8, 16, 32); }
     #undef AM_LDS
     #undef AM_LAUNCH

@@ -7,6 +7,8 @@
 // w, w + NW, ... (one key per lane, its row read in 16-byte pieces when the layout allows), keeps its own running maximum, sum and
 // value accumulators (MAXV = ceil(vdim / 64) per lane), and the waves are merged through LDS at the end.  Wave 0 starts from the sink.
 // The query's first dim1 elements are read from q, the rest from q2 (dim1 = dim: one part).  softcap > 0: score <- softcap tanh(score / softcap).
+// RowMap: where key j lies.  row_linear: row j.  row_jump: row j, and row j + jump from j = at on (the kept first tokens ahead of a window).  row_paged: through a
+// page table.  gate_row (optional): vdim gate values before their sigmoid, multiplied element by element with the result (`gate` is one factor for all).
 // TO: the element type of the result (float keeps the weighted sum unrounded for a caller that combines several maps).
 #define AT_WAVES 4
 
@@ -14,10 +16,25 @@ template <typename T> struct kvec;
 template <> struct kvec<bf16_t> { static constexpr int N = 8; };
 template <> struct kvec<float> { static constexpr int N = 4; };
 
-template <typename T, int MAXV, typename TO = T, int NW = AT_WAVES>
+struct row_linear
+{
+    __device__ __forceinline__ int64_t operator()(int j) const { return j; }
+};
+struct row_jump
+{
+    int at; int64_t jump;
+    __device__ __forceinline__ int64_t operator()(int j) const { return j < at ? (int64_t) j : j + jump; }
+};
+struct row_paged
+{
+    const int32_t* table; int page;
+    __device__ __forceinline__ int64_t operator()(int j) const { return (int64_t) table[j / page] * page + (j % page); }
+};
+
+template <typename T, int MAXV, typename TO = T, int NW = AT_WAVES, typename RowMap = row_linear>
 __device__ __forceinline__ void attn_row(TO* __restrict__ out, const T* __restrict__ q, const T* q2, int dim1, const T* __restrict__ kb, int64_t k_step, const T* __restrict__ vb,
                                          int64_t v_step, int count, int dim, int vdim, float scale, bool has_sink, float sink, float gate, bool k_vec,
-                                         float* smem, float softcap = 0.f)
+                                         float* smem, float softcap = 0.f, RowMap map = RowMap(), const T* gate_row = nullptr)
 {
     float* qs = smem;                                   // [dim]
     float* ps = qs + dim;                               // [NW][64]
@@ -38,7 +55,7 @@ __device__ __forceinline__ void attn_row(TO* __restrict__ out, const T* __restri
         float s = -INFINITY;
         if (j < count)
         {
-            const T* kr = kb + (int64_t) j * k_step;
+            const T* kr = kb + map(j) * k_step;
             float d = 0.f;
             if (k_vec)
             {
@@ -75,11 +92,11 @@ __device__ __forceinline__ void attn_row(TO* __restrict__ out, const T* __restri
                 {
                     float vv[8];
                     #pragma unroll
-                    for (int e = 0; e < 8; ++e) vv[e] = to_f(vb[(int64_t) (j0 + jj + e) * v_step + c]);
+                    for (int e = 0; e < 8; ++e) vv[e] = to_f(vb[map(j0 + jj + e) * v_step + c]);
                     #pragma unroll
                     for (int e = 0; e < 8; ++e) a += pw[jj + e] * vv[e];
                 }
-                for (; jj < cnt; ++jj) a += pw[jj] * to_f(vb[(int64_t) (j0 + jj) * v_step + c]);
+                for (; jj < cnt; ++jj) a += pw[jj] * to_f(vb[map(j0 + jj) * v_step + c]);
             }
             acc[i] = a;
         }
@@ -112,7 +129,7 @@ __device__ __forceinline__ void attn_row(TO* __restrict__ out, const T* __restri
     for (int i = 0; i < MAXV; ++i)
     {
         const int c = lane + 64 * i;
-        if (c < vdim) out[c] = from_f<TO>(acc[i] * f);
+        if (c < vdim) out[c] = from_f<TO>(acc[i] * f * (gate_row ? sigmoid_f(to_f(gate_row[c])) : 1.0f));
     }
 }
 

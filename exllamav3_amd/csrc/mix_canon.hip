@@ -35,10 +35,11 @@ template <typename T> __device__ __forceinline__ float rounded(float v) { return
 // into the ring at pos % (taps - 1).  Without conv_w, h = hn.  V: elements per thread and access (4 when the rows allow it).
 // CENTER: the norm is a layer norm, (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + bias, the mean taken first and the deviations squared after it.
 // y2 (optional): a second addend, y' = (y + y2) * y_scale (the two sublayers of a parallel block and the block's residual factor); without it y' = y * y_scale.
-// hn_out (optional): the normed row itself, for a consumer that reads it without the convolution.
+// hn_out (optional): the normed row itself, for a consumer that reads it without the convolution; with w2 (optional, RMS norm only) it is a SECOND norm of the
+// same row, x / sqrt(mean(x^2) + eps) * w2 -- two sublayers that each norm the same stream with a weight of their own read the statistics once.
 template <typename T, int V, bool CENTER>
 __global__ __launch_bounds__(CN_THREADS) void residual_rms_kernel(float* __restrict__ x, const T* __restrict__ y, int64_t y_ld, const T* __restrict__ y2, int64_t y2_ld, float y_scale,
-                                                                  int mode, const float* __restrict__ w, const float* __restrict__ bias, float eps,
+                                                                  int mode, const float* __restrict__ w, const float* __restrict__ w2, const float* __restrict__ bias, float eps,
                                                                   T* __restrict__ h, int64_t h_ld, T* __restrict__ hn_out, int64_t hn_ld,
                                                                   const float* __restrict__ conv_w, int taps, T* __restrict__ ring,
                                                                   const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
@@ -106,10 +107,19 @@ __global__ __launch_bounds__(CN_THREADS) void residual_rms_kernel(float* __restr
         }
         else
         {
+            if (w2)
+            {
+                float h2[V], wv2[V];
+                if constexpr (V == 4) { const float4 u = *(const float4*) (w2 + i); wv2[0] = u.x; wv2[1] = u.y; wv2[2] = u.z; wv2[V - 1] = u.w; } else wv2[0] = w2[i];
+                #pragma unroll
+                for (int e = 0; e < V; ++e) h2[e] = hn[e] * inv * wv2[e];
+                T* dst2 = hn_out + (int64_t) n * hn_ld + i;
+                if constexpr (V == 4) store4<T>(dst2, (const float (&)[4]) h2); else dst2[0] = from_f<T>(h2[0]);
+            }
             #pragma unroll
             for (int e = 0; e < V; ++e) hn[e] = rounded<T>(hn[e] * inv * wv[e]);        // the normed row is held in the activation type wherever it is kept
         }
-        if (hn_out)
+        if (hn_out && !w2)
         {
             T* dsth = hn_out + (int64_t) n * hn_ld + i;
             if constexpr (V == 4) store4<T>(dsth, (const float (&)[4]) hn); else dsth[0] = from_f<T>(hn[0]);
@@ -203,8 +213,8 @@ static bool rows_by_four(const void* p, int64_t ld, int dtype)
     return p == nullptr || ((uintptr_t) p % 16 == 0 && ld % (dtype == EXL3_MIX_BF16 ? 8 : 4) == 0);
 }
 
-extern "C" int exl3_mix_residual_norm_conv(float* x, const void* y, int64_t y_ld, const void* y2, int64_t y2_ld, float y_scale, int mode, int center, const float* w,
-                                           const float* bias, float eps, void* h, int64_t h_ld, void* hn_out, int64_t hn_ld, const float* conv_w, int taps, void* ring,
+static int residual_norm(float* x, const void* y, int64_t y_ld, const void* y2, int64_t y2_ld, float y_scale, int mode, int center, const float* w,
+                         const float* w2, const float* bias, float eps, void* h, int64_t h_ld, void* hn_out, int64_t hn_ld, const float* conv_w, int taps, void* ring,
                                            const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, int n, int width, int dtype, void* stream)
 {
     MIX_CHECK(x && n >= 0 && width > 0 && mode >= 0 && mode <= 2, "mix_residual_norm_conv: bad arguments");
@@ -212,14 +222,29 @@ extern "C" int exl3_mix_residual_norm_conv(float* x, const void* y, int64_t y_ld
     MIX_CHECK((!h && !hn_out) || (w && (!h || h_ld >= width) && (!hn_out || hn_ld >= width)), "mix_residual_norm_conv: the norm needs its weight");
     MIX_CHECK(center || !bias, "mix_residual_norm_conv: a bias goes with the layer norm");
     MIX_CHECK(!conv_w || (h && ring && tok_seq && tok_pos && slots && taps >= 1 && taps <= CN_MAX_TAPS), "mix_residual_norm_conv: the convolution needs 1..%d taps, the ring and the step's rows", CN_MAX_TAPS);
+    MIX_CHECK(!w2 || (h && hn_out && !center && !conv_w), "mix_residual_norm_pair: two RMS norms without a convolution");
     if (n == 0 || (mode == 0 && !h && !hn_out)) return EXL3_MIX_OK;
     const bool by4 = width % 8 == 0 && (uintptr_t) x % 16 == 0 && rows_by_four(y, y_ld, dtype) && rows_by_four(y2, y2_ld, dtype) && rows_by_four(h, h_ld, dtype) &&
-                     rows_by_four(hn_out, hn_ld, dtype) && rows_by_four(ring, 8, dtype) && (uintptr_t) w % 16 == 0 && (uintptr_t) conv_w % 16 == 0;
+                     rows_by_four(hn_out, hn_ld, dtype) && rows_by_four(ring, 8, dtype) && (uintptr_t) w % 16 == 0 && (uintptr_t) w2 % 16 == 0 && (uintptr_t) conv_w % 16 == 0;
     #define RN_LAUNCH(VV, CC) hipLaunchKernelGGL((residual_rms_kernel<T, VV, CC>), dim3(n), dim3(CN_THREADS), 0, (hipStream_t) stream, x, (const T*) y, y_ld, (const T*) y2, y2_ld, y_scale, \
-                                                 mode, w, bias, eps, (T*) h, h_ld, (T*) hn_out, hn_ld, conv_w, taps, (T*) ring, tok_seq, tok_pos, slots, width)
+                                                 mode, w, w2, bias, eps, (T*) h, h_ld, (T*) hn_out, hn_ld, conv_w, taps, (T*) ring, tok_seq, tok_pos, slots, width)
     MIX_DISPATCH_T(dtype, if (by4) { if (center) RN_LAUNCH(4, true); else RN_LAUNCH(4, false); } else { if (center) RN_LAUNCH(1, true); else RN_LAUNCH(1, false); });
     #undef RN_LAUNCH
     return mix_check_launch("mix_residual_norm_conv");
+}
+
+extern "C" int exl3_mix_residual_norm_conv(float* x, const void* y, int64_t y_ld, const void* y2, int64_t y2_ld, float y_scale, int mode, int center, const float* w,
+                                           const float* bias, float eps, void* h, int64_t h_ld, void* hn_out, int64_t hn_ld, const float* conv_w, int taps, void* ring,
+                                           const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, int n, int width, int dtype, void* stream)
+{
+    return residual_norm(x, y, y_ld, y2, y2_ld, y_scale, mode, center, w, nullptr, bias, eps, h, h_ld, hn_out, hn_ld, conv_w, taps, ring, tok_seq, tok_pos, slots, n, width, dtype, stream);
+}
+
+extern "C" int exl3_mix_residual_norm_pair(float* x, const void* y, int64_t y_ld, int mode, const float* w1, void* h1, int64_t h1_ld, const float* w2, void* h2, int64_t h2_ld,
+                                           float eps, int n, int width, int dtype, void* stream)
+{
+    return residual_norm(x, y, y_ld, nullptr, 0, 1.0f, mode, 0, w1, h2 ? w2 : nullptr, nullptr, eps, h1, h1_ld, h2, h2_ld, nullptr, 0, nullptr, nullptr, nullptr, nullptr, n, width, dtype,
+                         stream);
 }
 
 extern "C" int exl3_mix_residual_rms(float* x, const void* y, int64_t y_ld, int mode, const float* w, float eps, void* h, int64_t h_ld,

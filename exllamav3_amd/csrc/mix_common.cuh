@@ -65,16 +65,17 @@ __device__ __forceinline__ float block_sum(float v, float* red)
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
 // gated activations of two projections (g: gate, u: up).  EXL3_MIX_GLU_SILU: silu(g) u.  EXL3_MIX_GLU_CLAMPED_SWISH: g' = min(g, limit),
-// u' = clamp(u, -limit, limit), g' sigmoid(1.702 g') (u' + 1).
+// u' = clamp(u, -limit, limit), g' sigmoid(1.702 g') (u' + 1).  EXL3_MIX_GLU_GELU_TANH: gelu_tanh(g) u.
+__device__ __forceinline__ float gelu_tanh_f(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 __device__ __forceinline__ float glu_act_f(float g, float u, int kind, float limit)
 {
     if (kind == EXL3_MIX_GLU_SILU) return silu_f(g) * u;
+    if (kind == EXL3_MIX_GLU_GELU_TANH) return gelu_tanh_f(g) * u;
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     return g * sigmoid_f(1.702f * g) * (u + 1.0f);
 }
 // plain activations (EXL3_MIX_ACT_*): relu(z)^2, gelu in its tanh form, silu
-__device__ __forceinline__ float gelu_tanh_f(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 __device__ __forceinline__ float act_f(float v, int kind)
 {
     if (kind == EXL3_MIX_ACT_RELU2) { const float t = fmaxf(v, 0.f); return t * t; }

@@ -11,6 +11,10 @@
 //   latent_decode_mfma   the same on the matrix cores (bfloat16): all heads of a sequence score the SAME cached rows, so sixteen heads are the
 //                   sixteen columns of one MFMA tile and every cached row is read once per sixteen heads instead of once per head.  The keys of a
 //                   sequence are split over workgroups whose four waves share the rows' columns; a second kernel merges the partial sums (and adds the sink).
+//   latent_rows, rotate_heads   the same preparation for a layer without a window, whose rows live in the cache's PAGES: RMS norm of the latent and of a query
+//                   latent, the rotated key part (pairs of neighbours or of halves), the page rows; and the rotated part of every query head, which such a layer only
+//                   has after the query up-projection.  A layer that reads another layer's pages calls latent_rows for its query latent alone.
+//   The decode kernels take either a ring or pages (template); with pages the split length follows the sequence's length on the device.
 #include "mix_common.cuh"
 #include "mix_attn_row.cuh"
 
@@ -91,16 +95,111 @@ __global__ __launch_bounds__(256) void latent_fill_k_kernel(T* __restrict__ k, i
     }
 }
 
-template <typename T, int MAXV>
+// The pair of entries i of `half` in a rotated vector of 2 half entries
+__device__ __forceinline__ void pair_of(int i, int half, int interleaved, int& a, int& b) { a = interleaved ? 2 * i : i; b = interleaved ? 2 * i + 1 : i + half; }
+
+__device__ __forceinline__ void row_trig(float* trig, int pos, const float* __restrict__ freq, int half, float mag)
+{
+    for (int i = threadIdx.x; i < half; i += blockDim.x)
+    {
+        float sn, cs;
+        sincosf((float) pos * freq[i], &sn, &cs);
+        trig[2 * i] = cs * mag; trig[2 * i + 1] = sn * mag;
+    }
+}
+
+// One workgroup per row.  dkv (optional) [n][rank + rot_dim]: ckr[n] = [norm(latent) * kv_w | rotated key part], which also goes to the row's place in the
+// pages.  dq (optional) [n][q_rank]: cq[n] = norm(dq[n]) * q_w.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_rows_kernel(T* __restrict__ ckr, T* __restrict__ pages, const T* __restrict__ dkv, int64_t dkv_ld, const float* __restrict__ kv_w,
+                                                          T* __restrict__ cq, const T* __restrict__ dq, int64_t dq_ld, const float* __restrict__ q_w, int q_rank,
+                                                          const int32_t* __restrict__ table, int64_t table_ld, int page, const int32_t* __restrict__ tok_seq,
+                                                          const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ slots,
+                                                          const float* __restrict__ freq, float mag, int interleaved, float eps, int rot_dim, int rot_dims, int rank)
+{
+    __shared__ float red[4];
+    extern __shared__ float trig[];
+    const int n = blockIdx.x;
+    if (dq)
+    {
+        const T* src = dq + (int64_t) n * dq_ld;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < q_rank; i += 256) { const float v = to_f(src[i]); ss += v * v; }
+        ss = block_sum<4>(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float) q_rank + eps);
+        for (int i = threadIdx.x; i < q_rank; i += 256) cq[(int64_t) n * q_rank + i] = from_f<T>(to_f(src[i]) * inv * q_w[i]);
+    }
+    if (!dkv) return;
+    const int pos = tok_pos[n], row = rank + rot_dim, half = rot_dims / 2;
+    const int32_t* tb = table + (int64_t) slots[tok_seq[n]] * table_ld;
+    const T* src = dkv + (int64_t) n * dkv_ld;
+    T* dst = ckr + (int64_t) n * row;
+    T* pg = pages + ((int64_t) tb[pos / page] * page + (pos % page)) * row;
+    row_trig(trig, pos, freq, half, mag);
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < rank; i += 256) { const float v = to_f(src[i]); ss += v * v; }
+    ss = block_sum<4>(ss, red);                                // its barriers also publish trig
+    const float inv = 1.0f / sqrtf(ss / (float) rank + eps);
+    for (int i = threadIdx.x; i < rank; i += 256)
+    {
+        const T o = from_f<T>(to_f(src[i]) * inv * kv_w[i]);
+        dst[i] = o; pg[i] = o;
+    }
+    for (int i = threadIdx.x; i < half; i += 256)
+    {
+        int a, b;
+        pair_of(i, half, interleaved, a, b);
+        const float cs = trig[2 * i], sn = trig[2 * i + 1];
+        const float u = to_f(src[rank + a]), v = to_f(src[rank + b]);
+        const T o0 = from_f<T>(u * cs - v * sn), o1 = from_f<T>(v * cs + u * sn);
+        dst[rank + a] = o0; dst[rank + b] = o1;
+        pg[rank + a] = o0; pg[rank + b] = o1;
+    }
+    for (int i = rot_dims + threadIdx.x; i < rot_dim; i += 256) { const T o = src[rank + i]; dst[rank + i] = o; pg[rank + i] = o; }
+}
+
+// The rotated part of every query head, in place: entries off .. off + rot_dims of each of `heads` vectors of `step` elements
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_heads_kernel(T* __restrict__ q, int64_t q_ld, const int32_t* __restrict__ tok_pos, const float* __restrict__ freq, float mag,
+                                                           int interleaved, int heads, int step, int off, int rot_dims)
+{
+    extern __shared__ float trig[];
+    const int n = blockIdx.x, half = rot_dims / 2;
+    row_trig(trig, tok_pos[n], freq, half, mag);
+    __syncthreads();
+    T* qr = q + (int64_t) n * q_ld + off;
+    for (int t = threadIdx.x; t < heads * half; t += 256)
+    {
+        const int h = t / half, i = t - h * half;
+        int a, b;
+        pair_of(i, half, interleaved, a, b);
+        const float cs = trig[2 * i], sn = trig[2 * i + 1];
+        T* e = qr + (int64_t) h * step;
+        const float u = to_f(e[a]), v = to_f(e[b]);
+        e[a] = from_f<T>(u * cs - v * sn);
+        e[b] = from_f<T>(v * cs + u * sn);
+    }
+}
+
+// PAGED: the cached rows of a sequence lie in pages of `page` rows listed by its row of `table`; otherwise in the slot's ring of `window` rows
+template <typename T, int MAXV, bool PAGED>
 __global__ __launch_bounds__(64 * AT_WAVES) void latent_decode_kernel(T* __restrict__ o_lat, int64_t o_row, int64_t o_head, const T* __restrict__ q_lat, int64_t ql_row,
                                                                       int64_t ql_head, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ ring,
                                                                       const float* __restrict__ sink, const int32_t* __restrict__ slots,
-                                                                      const int32_t* __restrict__ len_after, int dim, int rot_dim, int rank, float scale, int window)
+                                                                      const int32_t* __restrict__ len_after, const int32_t* __restrict__ table, int64_t table_ld, int page, int dim, int rot_dim,
+                                                                      int rank, float scale, int window)
 {
     extern __shared__ float smem[];
     const int n = blockIdx.x, h = blockIdx.y;
-    const int count = min(len_after[n], window);
     const int row = rank + rot_dim;
+    if constexpr (PAGED)
+    {
+        attn_row<T, MAXV, T, AT_WAVES, row_paged>(o_lat + (int64_t) n * o_row + (int64_t) h * o_head, q_lat + (int64_t) n * ql_row + (int64_t) h * ql_head,
+                      q + (int64_t) n * q_ld + (int64_t) h * (dim + rot_dim) + dim, rank, ring, row, ring, row, len_after[n], row, rank, scale,
+                      sink != nullptr, sink ? sink[h] : 0.f, 1.0f, rows_are_16_byte(ring, (int64_t) row, row), smem, 0.f, row_paged{table + (int64_t) slots[n] * table_ld, page});
+        return;
+    }
+    const int count = min(len_after[n], window);
     const T* kb = ring + (int64_t) slots[n] * window * row;
     attn_row<T, MAXV>(o_lat + (int64_t) n * o_row + (int64_t) h * o_head, q_lat + (int64_t) n * ql_row + (int64_t) h * ql_head,
                       q + (int64_t) n * q_ld + (int64_t) h * (dim + rot_dim) + dim, rank, kb, row, kb, row, count, row, rank, scale,
@@ -130,23 +229,54 @@ extern "C" int exl3_mix_latent_fill_k(void* k, int64_t k_ld, const void* ckr, in
     return mix_check_launch("mix_latent_fill_k");
 }
 
+extern "C" int exl3_mix_latent_rows(void* ckr, void* pages, const void* dkv, int64_t dkv_ld, const float* kv_w, void* cq, const void* dq, int64_t dq_ld, const float* q_w,
+                                    int q_rank, const int32_t* table, int64_t table_ld, int page, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots,
+                                    const float* freq, float mag, int interleaved, float eps, int n, int rot_dim, int rot_dims, int rank, int dtype, void* stream)
+{
+    MIX_CHECK(n >= 0 && (dkv || dq), "mix_latent_rows: nothing to do");
+    MIX_CHECK(!dq || (cq && q_w && q_rank > 0 && dq_ld >= q_rank), "mix_latent_rows: bad query latent");
+    MIX_CHECK(!dkv || (ckr && pages && kv_w && table && tok_seq && tok_pos && slots && freq && rank > 0 && rot_dim >= 0 && dkv_ld >= rank + rot_dim && page > 0 && table_ld > 0),
+              "mix_latent_rows: bad latent");
+    MIX_CHECK(rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0 && rot_dims <= 8192, "mix_latent_rows: %d rotated dimensions of %d", rot_dims, rot_dim);
+    if (n == 0) return EXL3_MIX_OK;
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(latent_rows_kernel<T>, dim3(n), dim3(256), (size_t) (rot_dims + 2) * sizeof(float), (hipStream_t) stream, (T*) ckr, (T*) pages, (const T*) dkv,
+                                             dkv_ld, kv_w, (T*) cq, (const T*) dq, dq_ld, q_w, q_rank, table, table_ld, page, tok_seq, tok_pos, slots, freq, mag, interleaved, eps,
+                                             rot_dim, rot_dims, rank));
+    return mix_check_launch("mix_latent_rows");
+}
+
+extern "C" int exl3_mix_rotate_heads(void* q, int64_t q_ld, const int32_t* tok_pos, const float* freq, float mag, int interleaved, int n, int heads, int step, int off, int rot_dims,
+                                     int dtype, void* stream)
+{
+    MIX_CHECK(q && tok_pos && freq && n >= 0 && heads > 0 && step > 0 && off >= 0 && rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= 8192 && off + rot_dims <= step &&
+              q_ld >= (int64_t) heads * step, "mix_rotate_heads: bad arguments");
+    if (n == 0) return EXL3_MIX_OK;
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(rotate_heads_kernel<T>, dim3(n), dim3(256), (size_t) rot_dims * sizeof(float), (hipStream_t) stream, (T*) q, q_ld, tok_pos, freq, mag,
+                                             interleaved, heads, step, off, rot_dims));
+    return mix_check_launch("mix_rotate_heads");
+}
+
 extern "C" int exl3_mix_latent_decode(void* o_lat, int64_t o_row, int64_t o_head, const void* q_lat, int64_t ql_row, int64_t ql_head, const void* q, int64_t q_ld,
-                                      const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after,
+                                      const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after, const int32_t* table, int64_t table_ld, int page,
                                       int n, int heads, int dim, int rot_dim, int rank, float scale, int window, int dtype, void* stream)
 {
     MIX_CHECK(o_lat && q_lat && q && ring && slots && len_after, "mix_latent_decode: null pointer");
     MIX_CHECK(n >= 0 && heads > 0 && heads <= 65535 && dim >= 0 && rot_dim >= 0 && rank > 0 && rank <= 1024 && rank + rot_dim <= 4096 && window > 0,
               "mix_latent_decode: rank %d (<= 1024) / rot_dim %d / window %d out of range", rank, rot_dim, window);
     MIX_CHECK(q_ld >= (int64_t) heads * (dim + rot_dim), "mix_latent_decode: bad row stride");
+    MIX_CHECK(!table || (page > 0 && table_ld > 0), "mix_latent_decode: pages need their size and the table's row stride");
     if (n == 0) return EXL3_MIX_OK;
     const int mv = (rank + 63) / 64;
     const int mvt = mv == 1 ? 1 : (mv == 2 ? 2 : (mv <= 4 ? 4 : (mv <= 8 ? 8 : 16)));
     const size_t sm = (size_t) (rank + rot_dim + AT_WAVES * 64 + AT_WAVES * (2 + mvt * 64)) * sizeof(float);
-    #define LD_LAUNCH(MV) hipLaunchKernelGGL((latent_decode_kernel<T, MV>), dim3(n, heads), dim3(64 * AT_WAVES), sm, (hipStream_t) stream, (T*) o_lat, o_row, o_head, \
-                                             (const T*) q_lat, ql_row, ql_head, (const T*) q, q_ld, (const T*) ring, sink, slots, len_after, dim, rot_dim, rank, scale, window)
+    #define LD_LAUNCH_P(MV, PG) hipLaunchKernelGGL((latent_decode_kernel<T, MV, PG>), dim3(n, heads), dim3(64 * AT_WAVES), sm, (hipStream_t) stream, (T*) o_lat, o_row, o_head, \
+                                             (const T*) q_lat, ql_row, ql_head, (const T*) q, q_ld, (const T*) ring, sink, slots, len_after, table, table_ld, page, \
+                                             dim, rot_dim, rank, scale, window)
+    #define LD_LAUNCH(MV) do { if (table) LD_LAUNCH_P(MV, true); else LD_LAUNCH_P(MV, false); } while (0)
     MIX_DISPATCH_T(dtype,
         if (mv == 1) LD_LAUNCH(1); else if (mv == 2) LD_LAUNCH(2); else if (mv <= 4) LD_LAUNCH(4); else if (mv <= 8) LD_LAUNCH(8); else LD_LAUNCH(16));
     #undef LD_LAUNCH
+    #undef LD_LAUNCH_P
     return mix_check_launch("mix_latent_decode");
 }
 
@@ -168,12 +298,12 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 #define LM_VS (LM_KEYS + 8)
 #define LM_WAVES 4
 
-template <int NV>
+template <int NV, bool PAGED>
 __global__ __launch_bounds__(64 * LM_WAVES) void latent_decode_mfma_kernel(float* __restrict__ part_o, float* __restrict__ part_ml, const bf16_t* __restrict__ q_lat,
                                                                            int64_t ql_row, int64_t ql_head, const bf16_t* __restrict__ q, int64_t q_ld,
                                                                            const bf16_t* __restrict__ ring, const int32_t* __restrict__ slots,
                                                                            const int32_t* __restrict__ len_after, int heads, int dim, int rot_dim, int rank, float scale,
-                                                                           int window, int keys_per_split, int q_vec)
+                                                                           int window, int keys_per_split, int q_vec, const int32_t* __restrict__ table, int64_t table_ld, int page)
 {
     constexpr int KDW = NV / 8;                                 // 32-column steps of the padded latent per wave
     constexpr int NVW = NV / 4;                                 // 16-column tiles of the latent per wave
@@ -182,10 +312,12 @@ __global__ __launch_bounds__(64 * LM_WAVES) void latent_decode_mfma_kernel(float
     __shared__ __attribute__((aligned(16))) float sp[LM_WAVES][2][64][4];         // the waves' shares of the scores
     const int sp_i = blockIdx.x, hg = blockIdx.y, n = blockIdx.z, splits = gridDim.x;
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
-    const int count = min(len_after[n], window);
+    const int count = PAGED ? len_after[n] : min(len_after[n], window);
+    if (PAGED) keys_per_split = max(2 * LM_KEYS, ((count + splits - 1) / splits + LM_KEYS - 1) / LM_KEYS * LM_KEYS);
     const int k_begin = sp_i * keys_per_split, k_end = min(count, k_begin + keys_per_split);
     const int row = rank + rot_dim;
-    const bf16_t* kb = ring + (int64_t) slots[n] * window * row;
+    const bf16_t* kb = PAGED ? ring : ring + (int64_t) slots[n] * window * row;
+    const int32_t* tb = PAGED ? table + (int64_t) slots[n] * table_ld : nullptr;
     const int head = hg * 16 + c;
     const bool head_ok = head < heads;
     const int64_t pidx = ((int64_t) n * splits + sp_i) * heads + head;
@@ -227,7 +359,7 @@ __global__ __launch_bounds__(64 * LM_WAVES) void latent_decode_mfma_kernel(float
         for (int u = 0; u < 2; ++u)
         {
             const int jr = min(j0 + u * 16 + c, count - 1);       // rows past the split are read (they exist) and masked below
-            const bf16_t* kr = kb + (int64_t) jr * row;
+            const bf16_t* kr = kb + (PAGED ? (int64_t) tb[jr / page] * page + (jr % page) : (int64_t) jr) * row;
             #pragma unroll
             for (int i = 0; i < NS; ++i) kf[u][i].x = col_of[i] < row ? *(const uint4*) (kr + col_of[i]) : uint4{0u, 0u, 0u, 0u};
         }
@@ -350,7 +482,7 @@ extern "C" int exl3_mix_latent_decode_mfma_scratch(int n, int heads, int rank, i
 }
 
 extern "C" int exl3_mix_latent_decode_mfma(void* o_lat, int64_t o_row, int64_t o_head, const void* q_lat, int64_t ql_row, int64_t ql_head, const void* q, int64_t q_ld,
-                                           const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after, float* scratch, int splits,
+                                           const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after, const int32_t* table, int64_t table_ld, int page, float* scratch, int splits,
                                            int n, int heads, int dim, int rot_dim, int rank, float scale, int window, void* stream)
 {
     MIX_CHECK(o_lat && q_lat && q && ring && slots && len_after && scratch, "mix_latent_decode_mfma: null pointer");
@@ -359,6 +491,7 @@ extern "C" int exl3_mix_latent_decode_mfma(void* o_lat, int64_t o_row, int64_t o
     const int nv = rank <= 128 ? 8 : (rank <= 256 ? 16 : 32);
     MIX_CHECK(rank + rot_dim <= (nv / 2 + LM_WAVES) * 32, "mix_latent_decode_mfma: rot_dim %d too large beside rank %d", rot_dim, rank);
     MIX_CHECK((uintptr_t) ring % 16 == 0 && q_ld >= (int64_t) heads * (dim + rot_dim), "mix_latent_decode_mfma: the ring must be 16-byte aligned");
+    MIX_CHECK(!table || (page > 0 && table_ld > 0), "mix_latent_decode_mfma: pages need their size and the table's row stride");
     if (n == 0) return EXL3_MIX_OK;
     const int keys_per_split = (((window + splits - 1) / splits) + LM_KEYS - 1) / LM_KEYS * LM_KEYS;
     const int rp = nv * 16;
@@ -366,10 +499,13 @@ extern "C" int exl3_mix_latent_decode_mfma(void* o_lat, int64_t o_row, int64_t o
     float* part_o = scratch;
     float* part_ml = scratch + (int64_t) n * splits * heads * rp;
     const dim3 grid(splits, (heads + 15) / 16, n);
-    #define LM_LAUNCH(NVV) hipLaunchKernelGGL((latent_decode_mfma_kernel<NVV>), grid, dim3(64 * LM_WAVES), 0, (hipStream_t) stream, part_o, part_ml, (const bf16_t*) q_lat, ql_row, \
-                                              ql_head, (const bf16_t*) q, q_ld, (const bf16_t*) ring, slots, len_after, heads, dim, rot_dim, rank, scale, window, keys_per_split, q_vec)
+    #define LM_LAUNCH_P(NVV, PG) hipLaunchKernelGGL((latent_decode_mfma_kernel<NVV, PG>), grid, dim3(64 * LM_WAVES), 0, (hipStream_t) stream, part_o, part_ml, (const bf16_t*) q_lat, ql_row, \
+                                              ql_head, (const bf16_t*) q, q_ld, (const bf16_t*) ring, slots, len_after, heads, dim, rot_dim, rank, scale, window, keys_per_split, q_vec, table, \
+                                              table_ld, page)
+    #define LM_LAUNCH(NVV) do { if (table) LM_LAUNCH_P(NVV, true); else LM_LAUNCH_P(NVV, false); } while (0)
     if (nv == 8) LM_LAUNCH(8); else if (nv == 16) LM_LAUNCH(16); else LM_LAUNCH(32);
     #undef LM_LAUNCH
+    #undef LM_LAUNCH_P
     if (int rc = mix_check_launch("mix_latent_decode_mfma")) return rc;
     hipLaunchKernelGGL(latent_decode_merge_kernel, dim3(n, heads), dim3(128), (size_t) splits * sizeof(float), (hipStream_t) stream, (bf16_t*) o_lat, o_row, o_head, part_o, part_ml, sink, splits, heads, rank, rp);
     return mix_check_launch("mix_latent_decode_mfma (merge)");

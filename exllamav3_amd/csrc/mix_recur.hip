@@ -328,9 +328,9 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(float* __restrict__ qo,
     }
 }
 
-// out[n][h][i] = o[n][h][i] / sqrt(mean_i(o[n][h]^2) + eps) * w[(per_head ? h vdim : 0) + i] * gate(g[n][h vdim + i]); gate 0: silu, 1: sigmoid
+// out[n][h][i] = o[n][h][i] / sqrt(mean_i(o[n][h]^2) + eps) * w[(per_head ? h vdim : 0) + i] * gate(g[n][h vdim + i]); gate 0: silu, 1: sigmoid; w null: ones
 template <typename T>
-__global__ __launch_bounds__(64) void head_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ o, const float* __restrict__ w, int per_head, const T* __restrict__ g,
+__global__ __launch_bounds__(64) void head_norm_gate_kernel(T* __restrict__ out, int64_t out_ld, const float* __restrict__ o, const float* __restrict__ w, int per_head, const T* __restrict__ g,
                                                             int64_t g_ld, int gate, float eps, int heads, int vdim)
 {
     const int n = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -340,12 +340,12 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(T* __restrict__ out,
     ss = wave_sum(ss);
     const float inv = 1.0f / sqrtf(ss / (float) vdim + eps);
     const T* gr = g + (int64_t) n * g_ld + (int64_t) h * vdim;
-    const float* wr = w + (per_head ? (int64_t) h * vdim : 0);
-    T* dst = out + ((int64_t) n * heads + h) * vdim;
+    const float* wr = w ? w + (per_head ? (int64_t) h * vdim : 0) : nullptr;
+    T* dst = out + (int64_t) n * out_ld + (int64_t) h * vdim;
     for (int i = lane; i < vdim; i += 64)
     {
         const float z = to_f(gr[i]);
-        dst[i] = from_f<T>(orow[i] * inv * wr[i] * (gate == 0 ? silu_f(z) : sigmoid_f(z)));
+        dst[i] = from_f<T>(orow[i] * inv * (wr ? wr[i] : 1.0f) * (gate == 0 ? silu_f(z) : sigmoid_f(z)));
     }
 }
 
@@ -415,12 +415,12 @@ extern "C" int exl3_mix_delta_prep(float* qo, float* ko, float* vo, float* beta,
     return mix_check_launch("mix_delta_prep");
 }
 
-extern "C" int exl3_mix_head_norm_gate(void* out, const float* o, const float* w, int per_head, const void* g, int64_t g_ld, int gate, float eps, int n, int heads, int vdim,
+extern "C" int exl3_mix_head_norm_gate(void* out, int64_t out_ld, const float* o, const float* w, int per_head, const void* g, int64_t g_ld, int gate, float eps, int n, int heads, int vdim,
                                        int dtype, void* stream)
 {
-    MIX_CHECK(out && o && w && g && n >= 0 && heads > 0 && heads <= 65535 && vdim > 0 && g_ld >= (int64_t) heads * vdim && (gate == 0 || gate == 1), "mix_head_norm_gate: bad arguments");
+    MIX_CHECK(out && o && g && out_ld >= (int64_t) heads * vdim && n >= 0 && heads > 0 && heads <= 65535 && vdim > 0 && g_ld >= (int64_t) heads * vdim && (gate == 0 || gate == 1), "mix_head_norm_gate: bad arguments");
     if (n == 0) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(head_norm_gate_kernel<T>, dim3(n, heads), dim3(64), 0, (hipStream_t) stream, (T*) out, o, w, per_head, (const T*) g, g_ld, gate, eps, heads, vdim));
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(head_norm_gate_kernel<T>, dim3(n, heads), dim3(64), 0, (hipStream_t) stream, (T*) out, out_ld, o, w, per_head, (const T*) g, g_ld, gate, eps, heads, vdim));
     return mix_check_launch("mix_head_norm_gate");
 }
 

@@ -130,7 +130,7 @@ __global__ __launch_bounds__(256) void act_kernel(T* __restrict__ out, const T* 
 
 // rg (optional): one number per row; the row's result is multiplied by sigmoid(rg[n]) (a gate on the whole sublayer, applied before its linear down projection)
 template <typename T, bool VEC>
-__global__ __launch_bounds__(256) void glu_act_kernel(T* __restrict__ out, const T* __restrict__ g, int64_t g_ld, const T* __restrict__ u, int64_t u_ld, int ff, int kind, float limit,
+__global__ __launch_bounds__(256) void glu_act_kernel(T* __restrict__ out, int64_t out_ld, const T* __restrict__ g, int64_t g_ld, const T* __restrict__ u, int64_t u_ld, int ff, int kind, float limit,
                                                       const T* __restrict__ rg, int64_t rg_ld)
 {
     constexpr int VN = VEC ? rvec<T>::N : 1;
@@ -145,12 +145,12 @@ __global__ __launch_bounds__(256) void glu_act_kernel(T* __restrict__ out, const
         b.v = *(const uint4*) (u + (int64_t) n * u_ld + i);
         #pragma unroll
         for (int e = 0; e < rvec<T>::N; ++e) { const float r = glu_act_f(to_f(a.e[e]), to_f(b.e[e]), kind, limit); o.e[e] = from_f<T>(rg ? r * rs : r); }
-        *(uint4*) (out + (int64_t) n * ff + i) = o.v;
+        *(uint4*) (out + (int64_t) n * out_ld + i) = o.v;
     }
     else
     {
         const float r = glu_act_f(to_f(g[(int64_t) n * g_ld + i]), to_f(u[(int64_t) n * u_ld + i]), kind, limit);
-        out[(int64_t) n * ff + i] = from_f<T>(rg ? r * rs : r);
+        out[(int64_t) n * out_ld + i] = from_f<T>(rg ? r * rs : r);
     }
 }
 
@@ -169,7 +169,7 @@ __global__ __launch_bounds__(64) void token_gate_kernel(T* __restrict__ out, con
 
 // out[n][h * vdim + v] = a[n * a_row + h * a_head + v] * (gate ? sigmoid(gate[n][h * vdim + v]) : 1)
 template <typename T>
-__global__ __launch_bounds__(256) void heads_gate_kernel(T* __restrict__ out, const T* __restrict__ a, int64_t a_row, int64_t a_head, const T* __restrict__ gate,
+__global__ __launch_bounds__(256) void heads_gate_kernel(T* __restrict__ out, int64_t out_ld, const T* __restrict__ a, int64_t a_row, int64_t a_head, const T* __restrict__ gate,
                                                          int64_t gate_ld, int heads, int vdim)
 {
     const int n = blockIdx.x;
@@ -178,7 +178,7 @@ __global__ __launch_bounds__(256) void heads_gate_kernel(T* __restrict__ out, co
         const int h = t / vdim, v = t - h * vdim;
         float r = to_f(a[(int64_t) n * a_row + (int64_t) h * a_head + v]);
         if (gate) r *= sigmoid_f(to_f(gate[(int64_t) n * gate_ld + t]));
-        out[(int64_t) n * heads * vdim + t] = from_f<T>(r);
+        out[(int64_t) n * out_ld + t] = from_f<T>(r);
     }
 }
 
@@ -407,24 +407,24 @@ extern "C" int exl3_mix_act(void* out, const void* z, int64_t z_ld, int n, int f
 
 extern "C" int exl3_mix_glu_act(void* out, const void* g, int64_t g_ld, const void* u, int64_t u_ld, int n, int ff, int kind, float limit, int dtype, void* stream)
 {
-    return exl3_mix_glu_act_rowgate(out, g, g_ld, u, u_ld, nullptr, 0, n, ff, kind, limit, dtype, stream);
+    return exl3_mix_glu_act_rowgate(out, ff, g, g_ld, u, u_ld, nullptr, 0, n, ff, kind, limit, dtype, stream);
 }
 
-extern "C" int exl3_mix_glu_act_rowgate(void* out, const void* g, int64_t g_ld, const void* u, int64_t u_ld, const void* rg, int64_t rg_ld, int n, int ff, int kind, float limit,
+extern "C" int exl3_mix_glu_act_rowgate(void* out, int64_t out_ld, const void* g, int64_t g_ld, const void* u, int64_t u_ld, const void* rg, int64_t rg_ld, int n, int ff, int kind, float limit,
                                         int dtype, void* stream)
 {
-    MIX_CHECK(out && g && u && n >= 0 && ff > 0 && g_ld >= ff && u_ld >= ff && kind >= 0 && kind <= 1 && (!rg || rg_ld >= 1), "mix_glu_act: bad arguments");
+    MIX_CHECK(out && g && u && n >= 0 && ff > 0 && out_ld >= ff && g_ld >= ff && u_ld >= ff && kind >= 0 && kind <= 2 && (!rg || rg_ld >= 1), "mix_glu_act: bad arguments");
     const int vn = dtype == EXL3_MIX_BF16 ? 8 : 4;
-    const bool vec = ff % vn == 0 && g_ld % vn == 0 && u_ld % vn == 0 && (uintptr_t) out % 16 == 0 && (uintptr_t) g % 16 == 0 && (uintptr_t) u % 16 == 0;
+    const bool vec = ff % vn == 0 && out_ld % vn == 0 && g_ld % vn == 0 && u_ld % vn == 0 && (uintptr_t) out % 16 == 0 && (uintptr_t) g % 16 == 0 && (uintptr_t) u % 16 == 0;
     for (int r0 = 0; r0 < n; r0 += 65535)
     {
         const int rows = n - r0 < 65535 ? n - r0 : 65535;
         if (vec)
-            MIX_DISPATCH_T(dtype, hipLaunchKernelGGL((glu_act_kernel<T, true>), dim3((ff / vn + 255) / 256, rows), dim3(256), 0, (hipStream_t) stream, (T*) out + (int64_t) r0 * ff,
+            MIX_DISPATCH_T(dtype, hipLaunchKernelGGL((glu_act_kernel<T, true>), dim3((ff / vn + 255) / 256, rows), dim3(256), 0, (hipStream_t) stream, (T*) out + (int64_t) r0 * out_ld, out_ld,
                                                      (const T*) g + (int64_t) r0 * g_ld, g_ld, (const T*) u + (int64_t) r0 * u_ld, u_ld, ff, kind, limit,
                                                      rg ? (const T*) rg + (int64_t) r0 * rg_ld : nullptr, rg_ld));
         else
-            MIX_DISPATCH_T(dtype, hipLaunchKernelGGL((glu_act_kernel<T, false>), dim3((ff + 255) / 256, rows), dim3(256), 0, (hipStream_t) stream, (T*) out + (int64_t) r0 * ff,
+            MIX_DISPATCH_T(dtype, hipLaunchKernelGGL((glu_act_kernel<T, false>), dim3((ff + 255) / 256, rows), dim3(256), 0, (hipStream_t) stream, (T*) out + (int64_t) r0 * out_ld, out_ld,
                                                      (const T*) g + (int64_t) r0 * g_ld, g_ld, (const T*) u + (int64_t) r0 * u_ld, u_ld, ff, kind, limit,
                                                      rg ? (const T*) rg + (int64_t) r0 * rg_ld : nullptr, rg_ld));
     }
@@ -441,11 +441,11 @@ extern "C" int exl3_mix_token_gate(void* out, const void* gate, int64_t gate_ld,
     return mix_check_launch("mix_token_gate");
 }
 
-extern "C" int exl3_mix_heads_gate(void* out, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int n, int heads, int vdim, int dtype, void* stream)
+extern "C" int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int n, int heads, int vdim, int dtype, void* stream)
 {
-    MIX_CHECK(out && a && n >= 0 && heads > 0 && vdim > 0 && (!gate || gate_ld >= (int64_t) heads * vdim), "mix_heads_gate: bad arguments");
+    MIX_CHECK(out && a && n >= 0 && heads > 0 && vdim > 0 && out_ld >= (int64_t) heads * vdim && (!gate || gate_ld >= (int64_t) heads * vdim), "mix_heads_gate: bad arguments");
     if (n == 0) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(heads_gate_kernel<T>, dim3(n), dim3(256), 0, (hipStream_t) stream, (T*) out, (const T*) a, a_row, a_head, (const T*) gate, gate_ld,
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(heads_gate_kernel<T>, dim3(n), dim3(256), 0, (hipStream_t) stream, (T*) out, out_ld, (const T*) a, a_row, a_head, (const T*) gate, gate_ld,
                                              heads, vdim));
     return mix_check_launch("mix_heads_gate");
 }

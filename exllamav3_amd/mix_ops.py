@@ -248,7 +248,7 @@ def moe_vector_layout(h, ff: int) -> bool:
 
 
 # ---- pre-norm blocks with a statistics-free norm, gated activations, sigmoid router (csrc/mix_rowops.hip) ------------------------------------------
-GLU_SILU, GLU_CLAMPED_SWISH = 0, 1
+GLU_SILU, GLU_CLAMPED_SWISH, GLU_GELU_TANH = 0, 1, 2
 ACT_RELU2, ACT_GELU_TANH, ACT_SILU = 0, 1, 2
 RES_KEEP, RES_ADD, RES_SET = 0, 1, 2
 OUT_NONE, OUT_CAST, OUT_DYN_TANH = 0, 1, 2
@@ -302,9 +302,8 @@ def act(out: torch.Tensor, z_view: torch.Tensor, kind: int):
 
 
 def glu_act(out: torch.Tensor, g_view: torch.Tensor, u_view: torch.Tensor, kind: int, limit: float = 0.0):
-    n, ff = out.shape
-    _req(out.is_contiguous() and g_view.dtype == out.dtype == u_view.dtype and g_view.shape[0] == n and u_view.shape[0] == n, "glu_act: shapes")
-    _check(_lib.mixlib().exl3_mix_glu_act(_p(out), _p(g_view), _view(g_view, ff, "g"), _p(u_view), _view(u_view, ff, "u"), n, ff, kind, limit, code(out.dtype), _stream(out)))
+    """out may be a column block of a wider matrix."""
+    glu_act_rowgate(out, g_view, u_view, None, kind, limit)
 
 
 def token_gate(out: torch.Tensor, gate_view: torch.Tensor, table: torch.Tensor, col0: int, tokens: torch.Tensor):
@@ -319,10 +318,10 @@ def token_gate(out: torch.Tensor, gate_view: torch.Tensor, table: torch.Tensor, 
 def heads_gate(out: torch.Tensor, a: torch.Tensor, a_row: int, a_head: int, gate_view: torch.Tensor | None, heads: int, vdim: int):
     """a is addressed as base + n * a_row + h * a_head + v (token-major or head-major); the gate, if any, is [n, heads * vdim] before its sigmoid."""
     n = out.shape[0]
-    _req(out.is_contiguous() and out.shape == (n, heads * vdim) and a.dtype == out.dtype and a.numel() >= n * heads * vdim, "heads_gate: shapes")
+    _req(a.dtype == out.dtype and a.numel() >= n * heads * vdim, "heads_gate: shapes")
     if gate_view is not None:
         _req(gate_view.dtype == out.dtype and gate_view.shape[0] == n, "heads_gate: gate")
-    _check(_lib.mixlib().exl3_mix_heads_gate(_p(out), _p(a), a_row, a_head, _p(gate_view), 0 if gate_view is None else _view(gate_view, heads * vdim, "gate"), n, heads, vdim,
+    _check(_lib.mixlib().exl3_mix_heads_gate(_p(out), _view(out, heads * vdim, "out"), _p(a), a_row, a_head, _p(gate_view), 0 if gate_view is None else _view(gate_view, heads * vdim, "gate"), n, heads, vdim,
                                               code(out.dtype), _stream(out)))
 
 
@@ -413,9 +412,10 @@ def moe_gate_up_act(hid, h, wg, wu, idx, act_kind: int, limit: float):
 MASK_WINDOW, MASK_CHUNK = 0, 1
 
 
-def qk_prep(q_view, k_view, v_view, q_norm, k_norm, freq, mag: float, interleaved: bool, eps: float, ring_k, ring_v, tok_seq, tok_pos, slots, len_after, dim: int):
-    """In place on the step's queries and keys: RMS norm per (row, head, map) with a shared weight (None: no norm), rotary positions over 2 * len(freq)
-    leading entries (None: no rotation); keys and values of the rows a sequence keeps go into the rings."""
+def qk_prep(q_view, k_view, v_view, q_norm, k_norm, freq, mag: float, interleaved: bool, eps: float, ring_k, ring_v, tok_seq, tok_pos, slots, len_after, dim: int, k_out=None, keep_first: int = 0):
+    """In place on the step's queries and keys (keys into k_out if given: then k_view may be v_view itself): RMS norm per (row, head, map) with a shared weight (None: no norm), rotary positions over 2 * len(freq)
+    leading entries (None: no rotation); keys and values of the rows a sequence keeps go into the rings,
+    whose first `keep_first` entries hold the sequence's first positions for good."""
     n = q_view.shape[0]
     n_slots, window, k_heads, d2 = ring_k.shape
     v_heads, vdim = ring_v.shape[2], ring_v.shape[3]
@@ -430,35 +430,47 @@ def qk_prep(q_view, k_view, v_view, q_norm, k_norm, freq, mag: float, interleave
     if freq is not None:
         _f32c(freq, "freq")
     q_heads = q_view.shape[1] // dim
-    _req(tok_seq.numel() == n and tok_pos.numel() == n, "qk_prep: rows")
-    _check(_lib.mixlib().exl3_mix_qk_prep(_p(q_view), _view(q_view, q_heads * dim, "q"), _p(k_view), _view(k_view, k_heads * dim, "k"), _p(v_view),
-                                           _view(v_view, v_heads * vdim, "v"), _p(q_norm), _p(k_norm), _p(freq), 0 if freq is None else 2 * freq.numel(), mag,
+    k_dst = k_view if k_out is None else k_out
+    _req(tok_seq.numel() == n and tok_pos.numel() == n and k_dst.shape[0] == n and k_dst.dtype == k_view.dtype, "qk_prep: rows")
+    _check(_lib.mixlib().exl3_mix_qk_prep(_p(q_view), _view(q_view, q_heads * dim, "q"), _p(k_view), _view(k_view, k_heads * dim, "k"), _p(k_dst), _view(k_dst, k_heads * dim, "k_out"),
+                                           _p(v_view), _view(v_view, v_heads * vdim, "v"), _p(q_norm), _p(k_norm), _p(freq), 0 if freq is None else 2 * freq.numel(), mag,
                                            1 if interleaved else 0, eps, _p(ring_k), _p(ring_v), _p(tok_seq), _p(tok_pos), _p(slots), _p(len_after),
-                                           n, q_heads, k_heads, v_heads, dim, vdim, window, code(q_view.dtype), _stream(q_view)))
+                                           n, q_heads, k_heads, v_heads, dim, vdim, window, keep_first, code(q_view.dtype), _stream(q_view)))
+
+
+def _gate_args(gate_view, n: int, heads: int, vdim: int, dtype, name: str):
+    """A gate before its sigmoid: one column per head, or one per value element."""
+    if gate_view is None:
+        return None, 0, 1
+    cols = 1 if gate_view.shape[1] == heads else vdim
+    _req(gate_view.dtype == dtype and gate_view.shape[0] == n, f"{name}: gate")
+    return _p(gate_view), _view(gate_view, heads * cols, "gate"), cols
 
 
 def attn_prefill_maps(out, q_view, k_view, v_view, gate_view, sink, cu, tok_seq, tok_pos, heads: int, kv_heads: int, maps: int, dim: int, vdim: int, scale: float,
-                      softcap: float, window: int, mask: int, max_rows: int = 0, mfma: bool | None = None):
+                      softcap: float, window: int, mask: int, max_rows: int = 0, mfma: bool | None = None, keep: int = 0):
     """Prompt-step attention over the step's own keys with `maps` maps per head, a soft cap and a window or chunk mask.  out [n, heads * maps * vdim] in
-    float32 or the activation type.  mfma None: the matrix-core kernel for bfloat16 steps from ATTN_MFMA_MIN_ROWS rows."""
+    float32 or the activation type, possibly a column block of a wider matrix; the gate has one column per head or one per value element; the first `keep` positions
+    stay visible beside the window.  mfma None: the matrix-core kernel for bfloat16 steps from ATTN_MFMA_MIN_ROWS rows."""
     n = q_view.shape[0]
-    _req(out.is_contiguous() and out.shape == (n, heads * maps * vdim) and out.dtype in (torch.float32, q_view.dtype), "attn_prefill_maps: out")
+    out_ld = _view(out, heads * maps * vdim, "out")
+    _req(out.shape[0] == n and out.dtype in (torch.float32, q_view.dtype), "attn_prefill_maps: out")
     _req(q_view.dtype == k_view.dtype == v_view.dtype and k_view.shape[0] == n and v_view.shape[0] == n, "attn_prefill_maps: step tensors")
     if sink is not None:
         _f32c(sink, "sink"); _req(sink.numel() == heads and maps == 1, "attn_prefill_maps: sink")
     out_f32 = 1 if (out.dtype == torch.float32 and q_view.dtype != torch.float32) else 0
-    gate_ld = 0 if gate_view is None else _view(gate_view, heads, "gate")
+    gate, gate_ld, gate_cols = _gate_args(gate_view, n, heads, vdim, q_view.dtype, "attn_prefill_maps")
     if mfma is None:
         mfma = q_view.dtype == torch.bfloat16 and max_rows >= ATTN_MFMA_MIN_ROWS and dim <= 256 and vdim <= 256 and scale > 0
     if mfma:
         _req(q_view.dtype == torch.bfloat16 and max_rows > 0, "attn_prefill_maps: the matrix-core kernel takes bfloat16 and the step's longest sequence")
-        _check(_lib.mixlib().exl3_mix_attn_prefill_mfma_ex(_p(out), out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(k_view), _view(k_view, kv_heads * maps * dim, "k"),
-                                                            _p(v_view), _view(v_view, kv_heads * vdim, "v"), _p(gate_view), gate_ld, _p(sink), _p(cu), cu.numel() - 1, max_rows,
-                                                            heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, _stream(out)))
+        _check(_lib.mixlib().exl3_mix_attn_prefill_mfma_ex(_p(out), out_ld, out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(k_view), _view(k_view, kv_heads * maps * dim, "k"),
+                                                            _p(v_view), _view(v_view, kv_heads * vdim, "v"), gate, gate_ld, gate_cols, _p(sink), _p(cu), cu.numel() - 1, max_rows,
+                                                            heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, _stream(out)))
         return
-    _check(_lib.mixlib().exl3_mix_attn_prefill_ex(_p(out), out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(k_view), _view(k_view, kv_heads * maps * dim, "k"),
-                                                   _p(v_view), _view(v_view, kv_heads * vdim, "v"), _p(gate_view), gate_ld, _p(sink), _p(cu), _p(tok_seq), _p(tok_pos),
-                                                   n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, code(q_view.dtype), _stream(out)))
+    _check(_lib.mixlib().exl3_mix_attn_prefill_ex(_p(out), out_ld, out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(k_view), _view(k_view, kv_heads * maps * dim, "k"),
+                                                   _p(v_view), _view(v_view, kv_heads * vdim, "v"), gate, gate_ld, gate_cols, _p(sink), _p(cu), _p(tok_seq), _p(tok_pos),
+                                                   n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, code(q_view.dtype), _stream(out)))
 
 
 def diff_mfma_ok(dtype, max_rows: int, dim: int, vdim: int, scale: float) -> bool:
@@ -485,13 +497,15 @@ def attn_decode_maps(out, q_view, ring_k, ring_v, gate_view, sink, slots, len_af
     n_slots, window, k_heads, dim = ring_k.shape
     kv_heads, vdim = ring_v.shape[2], ring_v.shape[3]
     _req(k_heads == kv_heads * maps and ring_k.is_contiguous() and ring_v.is_contiguous() and ring_k.dtype == ring_v.dtype == q_view.dtype, "attn_decode_maps: rings")
-    _req(out.is_contiguous() and out.shape == (n, heads * maps * vdim) and out.dtype in (torch.float32, q_view.dtype), "attn_decode_maps: out")
+    out_ld = _view(out, heads * maps * vdim, "out")
+    gate, gate_ld, gate_cols = _gate_args(gate_view, n, heads, vdim, q_view.dtype, "attn_decode_maps")
+    _req(out.dtype in (torch.float32, q_view.dtype), "attn_decode_maps: out")
     _req(slots.numel() == n and len_after.numel() == n and q_view.shape[0] == n, "attn_decode_maps: one row per sequence")
     if sink is not None:
         _f32c(sink, "sink"); _req(sink.numel() == heads and maps == 1, "attn_decode_maps: sink")
     out_f32 = 1 if (out.dtype == torch.float32 and q_view.dtype != torch.float32) else 0
-    _check(_lib.mixlib().exl3_mix_attn_decode_ex(_p(out), out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(ring_k), _p(ring_v), _p(gate_view),
-                                                  0 if gate_view is None else _view(gate_view, heads, "gate"), _p(sink), _p(slots), _p(len_after),
+    _check(_lib.mixlib().exl3_mix_attn_decode_ex(_p(out), out_ld, out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(ring_k), _p(ring_v), gate,
+                                                  gate_ld, gate_cols, _p(sink), _p(slots), _p(len_after),
                                                   n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, code(q_view.dtype), _stream(out)))
 
 
@@ -693,13 +707,33 @@ def residual_norm_conv(x, y_view, y2_view, y_scale: float, mode: int, center: bo
                                                       n, width, code(ref.dtype), _stream(x)))
 
 
+def residual_norm_pair(x, y_view, mode: int, w1, h1_view, w2, h2_view, eps: float):
+    """x (float32, in place) = x | x + y | y; then h1 = rms_norm(x) w1 and (h2_view given) h2 = rms_norm(x) w2 over one pass of statistics.  h1_view None: the
+    update alone."""
+    n, width = x.shape
+    _f32c(x, "x")
+    ref = next((t for t in (y_view, h1_view) if t is not None), None)
+    _req(ref is not None, "residual_norm_pair: nothing to do")
+    if mode != RES_KEEP:
+        _req(y_view is not None and y_view.shape[0] == n, "residual_norm_pair: y")
+    else:
+        y_view = None
+    for h, w, nm in ((h1_view, w1, "h1"), (h2_view, w2, "h2")):
+        if h is not None:
+            _f32c(w, "w"); _req(w.numel() == width and h.shape[0] == n and h.dtype == ref.dtype, f"residual_norm_pair: {nm}")
+    _req(h1_view is not None or h2_view is None, "residual_norm_pair: the second norm comes beside the first")
+    ld = lambda t, nm: 0 if t is None else _view(t, width, nm)
+    _check(_lib.mixlib().exl3_mix_residual_norm_pair(_p(x), _p(y_view), ld(y_view, "y"), mode, _p(w1), _p(h1_view), ld(h1_view, "h1"), _p(w2) if h2_view is not None else None,
+                                                      _p(h2_view), ld(h2_view, "h2"), eps, n, width, code(ref.dtype), _stream(x)))
+
+
 def glu_act_rowgate(out: torch.Tensor, g_view: torch.Tensor, u_view: torch.Tensor, row_gate: torch.Tensor | None, kind: int, limit: float = 0.0):
     """out = glu(g, u) * sigmoid(row_gate[n]) (row_gate: [n, 1] view, one number per row)."""
     n, ff = out.shape
-    _req(out.is_contiguous() and g_view.dtype == out.dtype == u_view.dtype and g_view.shape[0] == n and u_view.shape[0] == n, "glu_act_rowgate: shapes")
+    _req(g_view.dtype == out.dtype == u_view.dtype and g_view.shape[0] == n and u_view.shape[0] == n, "glu_act_rowgate: shapes")
     if row_gate is not None:
         _req(row_gate.dtype == out.dtype and row_gate.shape == (n, 1), "glu_act_rowgate: the gate is one number per row")
-    _check(_lib.mixlib().exl3_mix_glu_act_rowgate(_p(out), _p(g_view), _view(g_view, ff, "g"), _p(u_view), _view(u_view, ff, "u"), _p(row_gate),
+    _check(_lib.mixlib().exl3_mix_glu_act_rowgate(_p(out), _view(out, ff, "out"), _p(g_view), _view(g_view, ff, "g"), _p(u_view), _view(u_view, ff, "u"), _p(row_gate),
                                                    0 if row_gate is None else max(row_gate.stride(0), 1), n, ff, kind, limit, code(out.dtype), _stream(out)))
 
 

@@ -37,6 +37,7 @@ extern "C" {
  * g' sigmoid(1.702 g') (u' + 1). */
 #define EXL3_MIX_GLU_SILU          0
 #define EXL3_MIX_GLU_CLAMPED_SWISH 1
+#define EXL3_MIX_GLU_GELU_TANH     2      /* gelu_tanh(g) u */
 /* plain activations */
 #define EXL3_MIX_ACT_RELU2     0
 #define EXL3_MIX_ACT_GELU_TANH 1
@@ -47,7 +48,7 @@ extern "C" {
 #define EXL3_MIX_MASK_WINDOW 0
 #define EXL3_MIX_MASK_CHUNK  1
 
-#define EXL3_MIX_ABI_VERSION 4
+#define EXL3_MIX_ABI_VERSION 5
 
 const char* exl3_mix_last_error(void);
 int  exl3_mix_abi_version(void);
@@ -168,7 +169,7 @@ int exl3_mix_token_gate(void* out, const void* gate, int64_t gate_ld, const void
 
 /* out[n][h * vdim + v] = a[n * a_row + h * a_head + v] * (gate ? sigmoid(gate[n][h * vdim + v]) : 1): an element-wise output gate over heads that may lie
  * head-major (the result of a per-head batched product). */
-int exl3_mix_heads_gate(void* out, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int n, int heads, int vdim, int dtype, void* stream);
+int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int n, int heads, int vdim, int dtype, void* stream);
 
 /* Router with independent scores s = sigmoid(z): the `top` experts with the largest s + correction (correction may be NULL; ties go to the lower index);
  * weights = s / (sum of the chosen s + 1e-20) * scale, or s * scale with normalise = 0. */
@@ -191,7 +192,7 @@ int exl3_mix_latent_fill_k(void* k, int64_t k_ld, const void* ckr, int n, int he
  * entries, softmax (with exp(sink_h) in the denominator if sink), o_lat = sum_j w_j c_j.  q_lat (the head's unrotated query carried into the latent space)
  * and o_lat are addressed as base + n * row_stride + h * head_stride; q_rot is read from q [n][heads][dim + rot_dim].  rank <= 1024. */
 int exl3_mix_latent_decode(void* o_lat, int64_t o_row, int64_t o_head, const void* q_lat, int64_t ql_row, int64_t ql_head, const void* q, int64_t q_ld,
-                           const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after,
+                           const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after, const int32_t* table, int64_t table_ld, int page,
                            int n, int heads, int dim, int rot_dim, int rank, float scale, int window, int dtype, void* stream);
 
 /* The same on the matrix cores, bfloat16 only: sixteen heads share every read of a cached row; the cached rows of a sequence are split over `splits`
@@ -199,8 +200,21 @@ int exl3_mix_latent_decode(void* o_lat, int64_t o_row, int64_t o_head, const voi
  * holds exl3_mix_latent_decode_mfma_scratch(...) floats. */
 int exl3_mix_latent_decode_mfma_scratch(int n, int heads, int rank, int splits, int64_t* floats);
 int exl3_mix_latent_decode_mfma(void* o_lat, int64_t o_row, int64_t o_head, const void* q_lat, int64_t ql_row, int64_t ql_head, const void* q, int64_t q_ld,
-                                const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after, float* scratch, int splits,
+                                const void* ring, const float* sink, const int32_t* slots, const int32_t* len_after, const int32_t* table, int64_t table_ld, int page, float* scratch, int splits,
                                 int n, int heads, int dim, int rot_dim, int rank, float scale, int window, void* stream);
+
+/* Both decode kernels with `table` (not NULL) read PAGES instead of a ring: `ring` is then the pool [pages][page][rank + rot_dim], a sequence of slot s owns the
+ * pages table[s * table_ld + 0, 1, ...] in order and all its len_after rows are visible (window is not used).
+ *
+ * What precedes them for such a layer, per row: dkv (may be NULL) [n][rank + rot_dim]: ckr[n] = [latent / rms * kv_w | key part rotated over its first rot_dims
+ * entries], stored in the row's page as well; dq (may be NULL) [n][q_rank]: cq[n] = dq[n] / rms * q_w (cq contiguous).  rotate_heads turns the entries
+ * off .. off + rot_dims of every one of `heads` vectors of `step` elements in place.  Pairs (i, i + rot_dims / 2), or (2i, 2i+1) when `interleaved`; angle = tok_pos *
+ * freq[i], cos and sin times mag. */
+int exl3_mix_latent_rows(void* ckr, void* pages, const void* dkv, int64_t dkv_ld, const float* kv_w, void* cq, const void* dq, int64_t dq_ld, const float* q_w,
+                         int q_rank, const int32_t* table, int64_t table_ld, int page, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots,
+                         const float* freq, float mag, int interleaved, float eps, int n, int rot_dim, int rot_dims, int rank, int dtype, void* stream);
+int exl3_mix_rotate_heads(void* q, int64_t q_ld, const int32_t* tok_pos, const float* freq, float mag, int interleaved, int n, int heads, int step, int off, int rot_dims,
+                          int dtype, void* stream);
 
 /* ---- several attention maps per head, chunk masks, soft-capped scores (mix_attn.hip, mix_attn_mfma.hip, mix_diffattn.hip) ---- */
 
@@ -208,15 +222,15 @@ int exl3_mix_latent_decode_mfma(void* o_lat, int64_t o_row, int64_t o_head, cons
  * of the head's key/value head; out [n][heads][maps][vdim]; a gate needs maps == 1), scores soft-capped to softcap tanh(score / softcap) (softcap 0: none),
  * mask EXL3_MIX_MASK_* over `window` positions, values as a column block (v_ld), and the result in float32 (out_f32) or the activation type.
  * Decode with the chunk mask reads the ring entries 0 .. (len_after - 1) % window. */
-int exl3_mix_attn_prefill_ex(void* out, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
-                             const void* gate, int64_t gate_ld, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
-                             int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int dtype, void* stream);
-int exl3_mix_attn_prefill_mfma_ex(void* out, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
-                                  const void* gate, int64_t gate_ld, const float* sink, const int32_t* cu,
-                                  int batch, int max_rows, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask,
+int exl3_mix_attn_prefill_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
+                             const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
+                             int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, int dtype, void* stream);
+int exl3_mix_attn_prefill_mfma_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
+                                  const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu,
+                                  int batch, int max_rows, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep,
                                   void* stream);
-int exl3_mix_attn_decode_ex(void* out, int out_f32, const void* q, int64_t q_ld, const void* ring_k, const void* ring_v,
-                            const void* gate, int64_t gate_ld, const float* sink, const int32_t* slots, const int32_t* len_after,
+int exl3_mix_attn_decode_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* ring_k, const void* ring_v,
+                            const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* slots, const int32_t* len_after,
                             int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int dtype, void* stream);
 
 /* Differential attention of a prompt step on the matrix cores, bfloat16 only: both maps of a head in one workgroup (the value tile is staged once for both)
@@ -231,10 +245,10 @@ int exl3_mix_attn_prefill_mfma_diff(void* out, const void* q, int64_t q_ld, cons
  * positions on the first rot_dims entries (freq [rot_dims / 2], NULL: none): pairs (i, i + rot_dims/2), or (2i, 2i+1) when `interleaved`; angle =
  * tok_pos * freq[i], cos and sin times `mag`.  q_heads and k_heads count every (head, map).  Keys and values of the rows with tok_pos >= len_after - window
  * go to ring_k [slots][window][k_heads][dim] and ring_v [slots][window][v_heads][vdim] at tok_pos % window. */
-int exl3_mix_qk_prep(void* q, int64_t q_ld, void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* q_norm, const float* k_norm,
+int exl3_mix_qk_prep(void* q, int64_t q_ld, const void* k, int64_t k_ld, void* k_out, int64_t ko_ld, const void* v, int64_t v_ld, const float* q_norm, const float* k_norm,
                      const float* freq, int rot_dims, float mag, int interleaved, float eps, void* ring_k, void* ring_v,
                      const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, const int32_t* len_after,
-                     int n, int q_heads, int k_heads, int v_heads, int dim, int vdim, int window, int dtype, void* stream);
+                     int n, int q_heads, int k_heads, int v_heads, int dim, int vdim, int window, int keep_first, int dtype, void* stream);
 
 /* Differential attention: a [n][heads][2][vdim] float32 (the two maps of every head);  o = a1 - lambda a2;
  * out[n][h][c] = o_c / sqrt(mean_c(o^2) + eps) * (1 - diff) * sigmoid(gate[n][h])  (gate NULL: no gate). */
@@ -296,8 +310,13 @@ int exl3_mix_residual_norm_conv(float* x, const void* y, int64_t y_ld, const voi
                                 const float* bias, float eps, void* h, int64_t h_ld, void* hn_out, int64_t hn_ld, const float* conv_w, int taps, void* ring,
                                 const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, int n, int width, int dtype, void* stream);
 
+/* The residual update of a block whose two sublayers each norm the same stream: x as in exl3_mix_residual_norm_conv (mode, one addend y), then
+ * u = x / sqrt(mean(x^2) + eps), h1 = u w1 and, if h2 is given, h2 = u w2.  h1 null: the update alone. */
+int exl3_mix_residual_norm_pair(float* x, const void* y, int64_t y_ld, int mode, const float* w1, void* h1, int64_t h1_ld, const float* w2, void* h2, int64_t h2_ld,
+                                float eps, int n, int width, int dtype, void* stream);
+
 /* exl3_mix_glu_act whose rows are also multiplied by sigmoid(rg[n]) (rg: one element per row, row stride rg_ld; may be null). */
-int exl3_mix_glu_act_rowgate(void* out, const void* g, int64_t g_ld, const void* u, int64_t u_ld, const void* rg, int64_t rg_ld, int n, int ff, int kind, float limit,
+int exl3_mix_glu_act_rowgate(void* out, int64_t out_ld, const void* g, int64_t g_ld, const void* u, int64_t u_ld, const void* rg, int64_t rg_ld, int n, int ff, int kind, float limit,
                              int dtype, void* stream);
 
 /* exl3_mix_topk_grouped with a group's score = the sum of its group_top largest choice scores (1: its largest). */
@@ -336,8 +355,20 @@ int exl3_mix_delta_scan(float* o, float* S_state, const float* q, const float* k
                         const int32_t* cu, const int32_t* slots, const int32_t* pos0, int batch, int heads, int kv_heads, int dim, int vdim, void* stream);
 
 /* out[n][h] = o[n][h] / rms(o[n][h]) * w[(per_head ? h vdim : 0) ..] * gate(g[n][h]); gate 0: silu, 1: sigmoid. */
-int exl3_mix_head_norm_gate(void* out, const float* o, const float* w, int per_head, const void* g, int64_t g_ld, int gate, float eps, int n, int heads, int vdim,
+int exl3_mix_head_norm_gate(void* out, int64_t out_ld, const float* o, const float* w, int per_head, const void* g, int64_t g_ld, int gate, float eps, int n, int heads, int vdim,
                             int dtype, void* stream);
+
+/* Retention (mix_retention.hip): per head S <- decay S + k v^T, o = S^T q with a fixed decay, q and k rotated (freq, rot_dims, interleaved as above; freq may be
+ * NULL with rot_dims 0) and k times k_scale.  pw [heads][pw_ld] = decay^0, decay^1, ... (at least 33 of them for the prompt form).  o [n][heads][vdim] float32,
+ * state [slots][heads][dim][vdim] float32, dim <= 256, vdim <= 1024.  segs > 1: every sequence in `segs` segments of seg_len rows that run in parallel; seg_state holds batch
+ * * segs * heads * dim * vdim floats. */
+int exl3_mix_retention(float* o, float* state, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* pw, int pw_ld,
+                       const float* freq, int rot_dims, int interleaved, const int32_t* cu, const int32_t* slots, const int32_t* pos0, int batch, int heads, int dim,
+                       int vdim, float k_scale, int segs, int seg_len, float* seg_state, int dtype, void* stream);
+/* One row per sequence, with what follows: out = o / rms(o per head) * silu(gate). */
+int exl3_mix_retention_step(void* out, int64_t out_ld, float* state, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
+                            const void* gate, int64_t gate_ld, const float* pw, int pw_ld, const float* freq, int rot_dims, int interleaved, const int32_t* tok_pos,
+                            const int32_t* slots, int n, int heads, int dim, int vdim, float k_scale, float eps, int dtype, void* stream);
 
 /* out[n] = scale (a[n] / rms(a[n]) * wa + b[n] / rms(b[n]) * wb). */
 int exl3_mix_rms_pair(void* out, const void* a, int64_t a_ld, const float* wa, const void* b, int64_t b_ld, const float* wb, float scale, float eps, int n, int width,
