@@ -367,11 +367,16 @@ def latent_mfma_ok(dtype, rank: int, rot_dim: int) -> bool:
 
 
 def latent_decode(o_lat: torch.Tensor, q_lat: torch.Tensor, q_view: torch.Tensor, ring: torch.Tensor, sink, slots, len_after, dim: int, rot_dim: int, scale: float,
-                  mfma: bool | None = None):
+                  mfma: bool | None = None, table: torch.Tensor | None = None):
     """o_lat, q_lat: [heads, n, rank] (any strides with a unit last one); q_view [n, heads * (dim + rot_dim)] holds the rotated parts.
+    ring: [slots, window, rank + rot_dim], or with `table` [slots, pages per slot] the pool of pages [pages, page, rank + rot_dim] (every row of a sequence visible).
     mfma None: the matrix-core kernel where it applies (bfloat16, rank and rot_dim multiples of 8, rank <= 512, rot_dim <= 128)."""
     heads, n, rank = q_lat.shape
     n_slots, window, row = ring.shape
+    tb, tb_ld, page = None, 0, 0
+    if table is not None:
+        _i32c(table, "page table")
+        tb, tb_ld, page = _p(table), table.stride(0), window
     if mfma is None:
         mfma = latent_mfma_ok(o_lat.dtype, rank, rot_dim)
     if mfma:
@@ -381,11 +386,12 @@ def latent_decode(o_lat: torch.Tensor, q_lat: torch.Tensor, q_view: torch.Tensor
         if sink is not None:
             _f32c(sink, "sink"); _req(sink.numel() == heads, "latent_decode: sink")
         groups = (heads + 15) // 16
-        splits = max(1, min(LATENT_MFMA_TARGET_WAVES // max(1, n * groups), (window + 63) // 64))
+        reach = table.shape[1] * page if table is not None else window                 # rows a sequence can have
+        splits = max(1, min(LATENT_MFMA_TARGET_WAVES // max(1, n * groups), (reach + 63) // 64))
         rp = 128 if rank <= 128 else (256 if rank <= 256 else 512)
         scratch = torch.empty(n * splits * heads * (rp + 2), dtype=torch.float32, device=o_lat.device)
         _check(_lib.mixlib().exl3_mix_latent_decode_mfma(_p(o_lat), o_lat.stride(1), o_lat.stride(0), _p(q_lat), q_lat.stride(1), q_lat.stride(0), _p(q_view),
-                                                          _view(q_view, heads * (dim + rot_dim), "q"), _p(ring), _p(sink), _p(slots), _p(len_after), _p(scratch), splits,
+                                                          _view(q_view, heads * (dim + rot_dim), "q"), _p(ring), _p(sink), _p(slots), _p(len_after), tb, tb_ld, page, _p(scratch), splits,
                                                           n, heads, dim, rot_dim, rank, scale, window, _stream(o_lat)))
         return
     _req(o_lat.shape == q_lat.shape and o_lat.stride(2) == 1 and q_lat.stride(2) == 1 and row == rank + rot_dim and ring.is_contiguous(), "latent_decode: shapes")
@@ -394,8 +400,46 @@ def latent_decode(o_lat: torch.Tensor, q_lat: torch.Tensor, q_view: torch.Tensor
     if sink is not None:
         _f32c(sink, "sink"); _req(sink.numel() == heads, "latent_decode: sink")
     _check(_lib.mixlib().exl3_mix_latent_decode(_p(o_lat), o_lat.stride(1), o_lat.stride(0), _p(q_lat), q_lat.stride(1), q_lat.stride(0), _p(q_view),
-                                                 _view(q_view, heads * (dim + rot_dim), "q"), _p(ring), _p(sink), _p(slots), _p(len_after), n, heads, dim, rot_dim, rank,
+                                                 _view(q_view, heads * (dim + rot_dim), "q"), _p(ring), _p(sink), _p(slots), _p(len_after), tb, tb_ld, page, n, heads, dim, rot_dim, rank,
                                                  scale, window, code(o_lat.dtype), _stream(o_lat)))
+
+
+def latent_rows(tok_seq, tok_pos, slots, eps: float, freq, mag: float, interleaved: bool, dkv=None, dq=None):
+    """The rows of a latent layer whose cache is paged.  dkv = (ckr [n, rank + rot_dim], pages [pages, page, rank + rot_dim], table, projection view, norm weight [rank]):
+    normed latent and rotated key part, into ckr and the row's page.  dq = (cq [n, q_rank], projection view, norm weight [q_rank]): normed query latent."""
+    _req(dkv is not None or dq is not None, "latent_rows: nothing to do")
+    n, dt = tok_seq.numel(), (dkv or dq)[0].dtype
+    kv = [None, None, None, 0, None]
+    tab, rot_dim, rot_dims, rank = (None, 0, 0), 0, 0, 0
+    for t, nm in ((tok_seq, "tok_seq"), (tok_pos, "tok_pos"), (slots, "slots")):
+        _i32c(t, nm)
+    _req(tok_pos.numel() == n, "latent_rows: rows")
+    if dkv is not None:
+        ckr, pages, table, z, w = dkv
+        _f32c(w, "latent norm"); _f32c(freq, "freq"); _i32c(table, "page table")
+        rank, rot_dims = w.numel(), 2 * freq.numel()
+        rot_dim = ckr.shape[1] - rank
+        _req(ckr.is_contiguous() and ckr.shape[0] == n and z.shape[0] == n and pages.is_contiguous() and pages.dim() == 3 and pages.shape[2] == rank + rot_dim
+             and ckr.dtype == pages.dtype == z.dtype and 0 <= rot_dims <= rot_dim, "latent_rows: latent shapes")
+        kv = [_p(ckr), _p(pages), _p(z), _view(z, rank + rot_dim, "dkv"), _p(w)]
+        tab = (_p(table), table.stride(0), pages.shape[1])
+    qa = [None, None, 0, None, 0]
+    if dq is not None:
+        cq, z, w = dq
+        _f32c(w, "query norm")
+        _req(cq.is_contiguous() and cq.shape == (n, w.numel()) and z.shape[0] == n and z.dtype == cq.dtype == dt, "latent_rows: query latent shapes")
+        qa = [_p(cq), _p(z), _view(z, w.numel(), "dq"), _p(w), w.numel()]
+    _check(_lib.mixlib().exl3_mix_latent_rows(*kv, *qa, *tab, _p(tok_seq), _p(tok_pos), _p(slots), _p(freq), mag, 1 if interleaved else 0, eps, n, rot_dim, rot_dims, rank,
+                                               code(dt), _stream(tok_seq)))
+
+
+def rotate_heads(q_view, tok_pos, freq, mag: float, interleaved: bool, heads: int, step: int, off: int):
+    """In place: entries off .. off + 2 len(freq) of every one of `heads` vectors of `step` entries per row turn with the row's position."""
+    n = q_view.shape[0]
+    _i32c(tok_pos, "tok_pos"); _f32c(freq, "freq")
+    _req(tok_pos.numel() == n, "rotate_heads: rows")
+    _check(_lib.mixlib().exl3_mix_rotate_heads(_p(q_view), _view(q_view, heads * step, "q"), _p(tok_pos), _p(freq), mag, 1 if interleaved else 0, n, heads, step, off,
+                                                2 * freq.numel(), code(q_view.dtype), _stream(q_view)))
 
 
 def moe_gate_up_act(hid, h, wg, wu, idx, act_kind: int, limit: float):
@@ -850,12 +894,15 @@ def delta_scan(o, S, q, k, v, beta, decay, cu, slots, pos0, kv_heads: int):
 
 
 def head_norm_gate(out, o, w, g_view, gate: int, eps: float):
-    """out [n, heads * vdim] = o / rms(o per head) * w * gate(g); w has vdim entries (shared by the heads) or heads * vdim; gate GATE_SILU / GATE_SIGMOID."""
+    """out [n, heads * vdim] = o / rms(o per head) * w * gate(g); w has vdim entries (shared by the heads) or heads * vdim, or is None
+    (ones); out may be a column block of a wider matrix; gate GATE_SILU / GATE_SIGMOID."""
     n, heads, vdim = o.shape
-    _f32c(o, "o"); _f32c(w, "w")
-    _req(out.is_contiguous() and out.shape == (n, heads * vdim) and w.numel() in (vdim, heads * vdim) and g_view.dtype == out.dtype, "head_norm_gate: shapes")
-    per_head = 1 if (w.numel() == heads * vdim and heads > 1) else 0
-    _check(_lib.mixlib().exl3_mix_head_norm_gate(_p(out), _p(o), _p(w), per_head, _p(g_view), _view(g_view, heads * vdim, "g"), gate, eps, n, heads, vdim, code(out.dtype),
+    _f32c(o, "o")
+    if w is not None:
+        _f32c(w, "w"); _req(w.numel() in (vdim, heads * vdim), "head_norm_gate: weight")
+    _req(out.shape[0] == n and g_view.dtype == out.dtype and g_view.shape[0] == n, "head_norm_gate: shapes")
+    per_head = 1 if (w is not None and w.numel() == heads * vdim and heads > 1) else 0
+    _check(_lib.mixlib().exl3_mix_head_norm_gate(_p(out), _view(out, heads * vdim, "out"), _p(o), _p(w), per_head, _p(g_view), _view(g_view, heads * vdim, "g"), gate, eps, n, heads, vdim, code(out.dtype),
                                                   _stream(out)))
 
 
@@ -867,3 +914,47 @@ def rms_pair(out, a_view, wa, b_view, wb, scale: float, eps: float):
          "rms_pair: shapes")
     _check(_lib.mixlib().exl3_mix_rms_pair(_p(out), _p(a_view), _view(a_view, width, "a"), _p(wa), _p(b_view), _view(b_view, width, "b"), _p(wb), scale, eps, n, width,
                                             code(out.dtype), _stream(out)))
+
+
+# ---- retention: linear attention with a fixed decay per head (csrc/mix_retention.hip) ----------------------------------------------------------------
+RETENTION_TILE = 32           # rows of a prompt tile: the table of powers holds decay^0 .. decay^RETENTION_TILE
+
+
+def _retention_args(q_view, k_view, v_view, pw, freq, heads: int, dim: int, vdim: int, name: str):
+    _f32c(pw, "pw")
+    if freq is not None:
+        _f32c(freq, "freq")
+    _req(pw.dim() == 2 and pw.shape[0] == heads and pw.shape[1] > RETENTION_TILE and q_view.dtype == k_view.dtype == v_view.dtype
+         and q_view.shape[0] == k_view.shape[0] == v_view.shape[0], f"{name}: shapes")
+    rot_dims = 0 if freq is None else 2 * freq.numel()
+    return (_p(q_view), _view(q_view, heads * dim, "q"), _p(k_view), _view(k_view, heads * dim, "k"), _p(v_view), _view(v_view, heads * vdim, "v")), \
+        (_p(pw), pw.shape[1], _p(freq), rot_dims)
+
+
+def retention(o, state, q_view, k_view, v_view, pw, freq, interleaved: bool, cu, slots, pos0, k_scale: float, segments: tuple[int, int] | None = None):
+    """Prompt steps: o [n, heads, vdim] float32, state [slots, heads, dim, vdim] float32; pw [heads, > RETENTION_TILE] float32 = powers of each head's decay; freq: the
+    rotation's frequencies.  segments = (segs, seg_len): every sequence cut into parallel segments; None: one chain of tiles per sequence."""
+    n, heads, vdim = o.shape
+    dim = state.shape[2]
+    _f32c(o, "o"); _f32c(state, "state")
+    for t, nm in ((cu, "cu"), (slots, "slots"), (pos0, "pos0")):
+        _i32c(t, nm)
+    batch = slots.numel()
+    _req(state.shape[1:] == (heads, dim, vdim) and cu.numel() == batch + 1 and pos0.numel() == batch and q_view.shape[0] == n, "retention: shapes")
+    a, b = _retention_args(q_view, k_view, v_view, pw, freq, heads, dim, vdim, "retention")
+    segs, seg_len = segments or (1, 0)
+    seg_state = torch.empty((batch * segs, heads, dim, vdim), dtype=torch.float32, device=o.device) if segs > 1 else None
+    _check(_lib.mixlib().exl3_mix_retention(_p(o), _p(state), *a, *b, 1 if interleaved else 0, _p(cu), _p(slots), _p(pos0), batch, heads, dim, vdim, k_scale, segs, seg_len,
+                                             _p(seg_state), code(q_view.dtype), _stream(o)))
+
+
+def retention_step(out, state, q_view, k_view, v_view, gate_view, pw, freq, interleaved: bool, tok_pos, slots, heads: int, k_scale: float, eps: float):
+    """One row per sequence: state update, read-out, head norm and silu gate in one launch; out [n, heads * vdim], possibly a column block of a wider matrix."""
+    n = out.shape[0]
+    dim, vdim = state.shape[2], state.shape[3]
+    _f32c(state, "state"); _i32c(tok_pos, "tok_pos"); _i32c(slots, "slots")
+    _req(state.shape[1] == heads and slots.numel() == n and tok_pos.numel() == n and q_view.shape[0] == n and gate_view.shape[0] == n
+         and gate_view.dtype == out.dtype == q_view.dtype, "retention_step: shapes")
+    a, b = _retention_args(q_view, k_view, v_view, pw, freq, heads, dim, vdim, "retention_step")
+    _check(_lib.mixlib().exl3_mix_retention_step(_p(out), _view(out, heads * vdim, "out"), _p(state), *a, _p(gate_view), _view(gate_view, heads * vdim, "gate"), *b,
+                                                  1 if interleaved else 0, _p(tok_pos), _p(slots), n, heads, dim, vdim, k_scale, eps, code(out.dtype), _stream(out)))

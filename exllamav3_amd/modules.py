@@ -37,6 +37,13 @@ float32 accumulation; true float32 when the model runs in float32).
     GatedDeltaRule          delta-rule memory with a scalar decay per head and token, short convolutions with silu on q / k / v, unit query / key vectors
     ParallelMixer           two mixers side by side over ONE fused input product, their outputs RMS-normed and averaged
     ParallelBlock           x += m (mixer(conv(n(x))) + ff(n(x))): one norm, both sublayers read it, the residual factor m
+    PagedLatentAttention    latent attention without a window: the cached rows live in the cache's pages; queries through a normed latent of their own; either
+                            pairing of the rotation; a layer may read another layer's cached rows instead of having any
+    KeptWindowAttention     grouped-query attention over a sliding window beside which the first tokens of a sequence stay visible; rotated queries and keys, values
+                            of their own or the keys before their rotation; sink, output gate per value element
+    Retention               linear attention with a fixed decay per head, rotated queries and keys, float32 state, per-head unit RMS, silu gate
+    DualNormBlock           x += mixer(norm1(x)) + ff(norm2(x)): both norms from one pass over the stream, both output projections as ONE product over
+                            [mixer's heads | hidden activation]
 
 Every sum that the model's exactness rests on (norms, scores, softmax, decays, states, the residual) is float32 inside the kernels in
 both modes; the element type only decides how matrix products and their outputs are held.
@@ -46,7 +53,7 @@ from dataclasses import dataclass
 import torch
 import torch.nn.functional as F
 from . import mix_ops
-from .state_cache import StateSpec, StepBatch
+from .state_cache import PagedSpec, StateSpec, StepBatch
 
 
 def _w(stc, key: str, dtype, device) -> torch.Tensor:
@@ -259,9 +266,12 @@ class LatentAttention:
             parts.append(("g", _w(stc, prefix + "g", dtype, device), None))
         self.inp = FusedInput(parts + list(extra_parts))
         self.c_norm = _f32(stc, prefix + "dkv.norm", device)
+        assert self.inp.offsets["q"][1] == self.heads * self.qk and self.inp.offsets["dkv"][1] == self.rank + self.rot_dim
+        self._load_up(stc, prefix, dtype, device)
+
+    def _load_up(self, stc, prefix: str, dtype, device):
         w_uk, self.w_uv = _w(stc, prefix + "uk", dtype, device), _w(stc, prefix + "uv", dtype, device)
         H, d, r, dv, rank = self.heads, self.dim, self.rot_dim, self.vdim, self.rank
-        assert self.inp.offsets["q"][1] == H * self.qk and self.inp.offsets["dkv"][1] == rank + r
         assert w_uk.shape == (H * d, rank) and self.w_uv.shape == (H * dv, rank)
         # prompt steps: keys of all heads as ONE product whose result already has room for the rotated part behind every head (zero weight rows there)
         padded = torch.zeros((H, self.qk, rank), dtype=dtype, device=device)
@@ -269,7 +279,7 @@ class LatentAttention:
         self.w_uk_padded = padded.view(H * self.qk, rank)
         # decode steps, absorbed form: per head q_lat = q_unrotated W_uk[h] and o = o_lat W_uv[h]^T
         self.w_uk_heads = w_uk.view(H, d, rank)
-        self.w_uv_heads_t = self.w_uv.view(H, dv, rank).transpose(1, 2)
+        self.w_uv_heads_t = self.w_uv.view(H, dv, rank).transpose(1, 2).contiguous()
         self.sink = _f32(stc, prefix + "sink", device) if self.has_sink else None
         self.w_o = _w(stc, prefix + "o", dtype, device)
         assert self.w_o.shape == (self.width, H * dv)
@@ -312,6 +322,184 @@ class LatentAttention:
         return F.linear(out, self.w_o), p
 
 
+class PagedLatentAttention(LatentAttention):
+    """Latent attention over every earlier token.  Queries pass a latent too: c_q = RMSnorm(W_dq h), q = W_uq c_q; [normed latent | rotated key part] of every token
+    lives in the cache's pages.  kv_from: the layer whose rows this layer reads (it has no W_dkv and stores nothing): in prompt steps that layer's rows
+    of the same step, handed over in the step's `shared` dict, in decode steps that layer's pages."""
+
+    def __init__(self, width: int, heads: int, dim: int, rot_dim: int, vdim: int, rank: int, q_rank: int, scale: float, eps: float, rot_dims: int, rot_base: float,
+                 rot_scaling: dict | None = None, interleaved: bool = False, sink: bool = False, gate: bool = False, layer: int = 0, kv_from: int | None = None):
+        super().__init__(width, heads, dim, rot_dim, vdim, rank, scale, 1, eps, rot_dims, rot_base, rot_scaling, sink, gate)
+        self.q_rank, self.interleaved, self.layer, self.kv_from = int(q_rank), bool(interleaved), layer, kv_from
+        self.out_width = heads * vdim
+
+    EVERY = 1 << 30                          # a window that no sequence reaches the end of
+
+    def load(self, stc, prefix: str, dtype, device, extra_parts=()):
+        parts = [("dq", _w(stc, prefix + "dq", dtype, device), None)]
+        if self.kv_from is None:
+            parts.append(("dkv", _w(stc, prefix + "dkv", dtype, device), None))
+        if self.has_gate:
+            parts.append(("g", _w(stc, prefix + "g", dtype, device), None))
+        self.inp = FusedInput(parts + list(extra_parts))
+        self.q_norm, self.w_uq = _f32(stc, prefix + "dq.norm", device), _w(stc, prefix + "uq", dtype, device)
+        assert self.inp.offsets["dq"][1] == self.q_rank == self.q_norm.numel() and self.w_uq.shape == (self.heads * self.qk, self.q_rank)
+        if self.kv_from is None:
+            self.c_norm = _f32(stc, prefix + "dkv.norm", device)
+            assert self.inp.offsets["dkv"][1] == self.rank + self.rot_dim and self.c_norm.numel() == self.rank
+        self._load_up(stc, prefix, dtype, device)
+
+    def state_specs(self) -> list:
+        return [] if self.kv_from is not None else [PagedSpec("latent", (self.rank + self.rot_dim,), self.dtype)]
+
+    def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
+        """out [n, heads * vdim]: the gated heads before the output projection.  state: this layer's, or that of the layer whose rows it reads."""
+        H, d, r, dv, rank = self.heads, self.dim, self.rot_dim, self.vdim, self.rank
+        p = self.inp(h)
+        pages, table = state["latent"], state["page_table"]
+        cq = torch.empty((sb.n, self.q_rank), dtype=self.dtype, device=h.device)
+        dkv = None
+        if self.kv_from is None:
+            ckr = torch.empty((sb.n, rank + r), dtype=self.dtype, device=h.device)
+            dkv = (ckr, pages, table, p["dkv"], self.c_norm)
+            if not sb.decode:
+                sb.shared["latent", self.layer] = ckr
+        mix_ops.latent_rows(sb.tok_seq, sb.tok_pos, sb.slots, self.eps, self.freq, self.rot_mag, self.interleaved, dkv=dkv, dq=(cq, p["dq"], self.q_norm))
+        q = F.linear(cq, self.w_uq)
+        if self.rot_dims:
+            mix_ops.rotate_heads(q, sb.tok_pos, self.freq, self.rot_mag, self.interleaved, H, self.qk, d)
+        if sb.decode:
+            q_heads = q.as_strided((H, sb.n, d), (self.qk, q.stride(0), 1), q.storage_offset())
+            q_lat = torch.bmm(q_heads, self.w_uk_heads)                          # [H, n, rank]
+            o_lat = torch.empty_like(q_lat)
+            mix_ops.latent_decode(o_lat, q_lat, q, pages, self.sink, sb.slots, sb.len_after, d, r, self.scale, table=table)
+            o = torch.bmm(o_lat, self.w_uv_heads_t)                              # [H, n, vdim]
+            mix_ops.heads_gate(out, o, dv, sb.n * dv, p.get("g"), H, dv)
+            return
+        ckr = sb.shared["latent", self.layer if self.kv_from is None else self.kv_from]
+        c = ckr[:, :rank]
+        k = F.linear(c, self.w_uk_padded)                                        # [n, H * (d + r)], the rotated slots still zero
+        v = F.linear(c, self.w_uv)
+        mix_ops.latent_fill_k(k, ckr, H, d, r, rank)
+        mix_ops.attn_prefill_maps(out, q, k, v, p.get("g"), self.sink, sb.cu, sb.tok_seq, sb.tok_pos, H, H, 1, self.qk, dv, self.scale, 0.0, self.EVERY, mix_ops.MASK_WINDOW,
+                                  max_rows=sb.max_rows)
+
+    def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
+        out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
+        self.attend(h, sb, state, out)
+        return F.linear(out, self.w_o)
+
+
+class KeptWindowAttention:
+    """H query heads over G key/value heads, no biases.  A row sees the last `size` positions up to itself and the sequence's first `keep_first` positions, which keep
+    their true positions.  Rotary positions on the first rot_dims entries of queries and keys; tied: the values are the keys before their rotation (no W_v).
+    Optional sink (one more term of the denominator per head) and output gate per value element.  A slot holds keep_first + size rows of keys and values: the
+    first positions' for good, and a ring of the last `size` of the others."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, size: int, keep_first: int, rot_dims: int, rot_base: float,
+                 interleaved: bool = True, tied: bool = False, sink: bool = True, gate: bool = True):
+        if heads % kv_heads:
+            raise RuntimeError(f"attention: {heads} query heads over {kv_heads} key/value heads")
+        if tied and dim != vdim:
+            raise RuntimeError(f"attention: values that are the keys have their size ({dim}, not {vdim})")
+        if rot_dims > dim or rot_dims % 2 or size < 1 or keep_first < 0:
+            raise RuntimeError(f"attention: {rot_dims} rotated dimensions of {dim}, a window of {size} beside {keep_first} first tokens")
+        self.width, self.heads, self.kv_heads, self.dim, self.vdim, self.scale = width, heads, kv_heads, dim, vdim, float(scale)
+        self.size, self.keep_first, self.rot_dims, self.rot_base, self.interleaved = int(size), int(keep_first), int(rot_dims), float(rot_base), bool(interleaved)
+        self.tied, self.has_sink, self.has_gate = tied, sink, gate
+        self.out_width = heads * vdim
+
+    def load(self, stc, prefix: str, dtype, device, extra_parts=()):
+        names = ["q", "k"] + ([] if self.tied else ["v"]) + (["g"] if self.has_gate else [])
+        self.inp = FusedInput([(nm, _w(stc, prefix + nm, dtype, device), None) for nm in names] + list(extra_parts))
+        self.sink = _f32(stc, prefix + "sink", device) if self.has_sink else None
+        self.w_o = _w(stc, prefix + "o", dtype, device)
+        assert self.inp.offsets["q"][1] == self.heads * self.dim and self.inp.offsets["k"][1] == self.kv_heads * self.dim
+        assert self.w_o.shape == (self.width, self.out_width)
+        self.freq = rotary_frequencies(self.rot_dims, self.rot_base)[0].to(device).contiguous() if self.rot_dims else None
+        self.dtype = dtype
+
+    def state_specs(self) -> list:
+        rows = self.keep_first + self.size
+        return [StateSpec("ring_k", (rows, self.kv_heads, self.dim), self.dtype), StateSpec("ring_v", (rows, self.kv_heads, self.vdim), self.dtype)]
+
+    def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
+        H, G, d, dv = self.heads, self.kv_heads, self.dim, self.vdim
+        p = self.inp(h)
+        q, k = p["q"], p["k"]
+        v = k if self.tied else p["v"]
+        k_rot = torch.empty((sb.n, G * d), dtype=self.dtype, device=h.device) if self.tied else None
+        mix_ops.qk_prep(q, k, v, None, None, self.freq, 1.0, self.interleaved, 0.0, state["ring_k"], state["ring_v"], sb.tok_seq, sb.tok_pos, sb.slots, sb.len_after, d,
+                        k_out=k_rot, keep_first=self.keep_first)
+        if sb.decode:
+            mix_ops.attn_decode_maps(out, q, state["ring_k"], state["ring_v"], p.get("g"), self.sink, sb.slots, sb.len_after, H, 1, self.scale, 0.0, mix_ops.MASK_WINDOW)
+        else:
+            mix_ops.attn_prefill_maps(out, q, k_rot if self.tied else k, v, p.get("g"), self.sink, sb.cu, sb.tok_seq, sb.tok_pos, H, G, 1, d, dv, self.scale, 0.0, self.size,
+                                      mix_ops.MASK_WINDOW, max_rows=sb.max_rows, keep=self.keep_first)
+
+    def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
+        out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
+        self.attend(h, sb, state, out)
+        return F.linear(out, self.w_o)
+
+
+class Retention:
+    """Per head S <- decay S + k v^T, o = S^T q with a fixed decay; q and k rotated over their first rot_dims entries, k times dim^(-1/2) after the rotation; each
+    head's o over its root mean square (no weight), times silu(W_g h).  State per slot: S [heads, dim, vdim] float32."""
+    # prompt steps whose longest sequence has at least this many rows are cut into parallel segments, enough of them for about this many workgroups
+    SEGMENT_MIN_ROWS = 256
+    SEGMENT_TARGET_WORKGROUPS = 1024
+    SEGMENT_ROWS = 64                        # a segment's shortest length
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay, rot_dims: int, rot_base: float, eps: float, interleaved: bool = False):
+        if len(decay) != heads:
+            raise RuntimeError(f"retention: {len(decay)} decays for {heads} heads")
+        if rot_dims > dim or rot_dims % 2:
+            raise RuntimeError(f"retention: {rot_dims} rotated dimensions of {dim}")
+        self.width, self.heads, self.dim, self.vdim, self.eps = width, heads, dim, vdim, float(eps)
+        self.decay, self.rot_dims, self.rot_base, self.interleaved = [float(x) for x in decay], int(rot_dims), float(rot_base), bool(interleaved)
+        self.k_scale = float(dim) ** -0.5
+        self.out_width = heads * vdim
+
+    def load(self, stc, prefix: str, dtype, device, extra_parts=()):
+        self.inp = FusedInput([(nm, _w(stc, prefix + nm, dtype, device), None) for nm in ("q", "k", "v", "g")] + list(extra_parts))
+        self.w_o = _w(stc, prefix + "o", dtype, device)
+        assert self.inp.offsets["q"][1] == self.inp.offsets["k"][1] == self.heads * self.dim and self.inp.offsets["v"][1] == self.out_width == self.inp.offsets["g"][1]
+        assert self.w_o.shape == (self.width, self.out_width)
+        powers = torch.arange(mix_ops.RETENTION_TILE + 1, dtype=torch.float64)
+        self.pw = (torch.tensor(self.decay, dtype=torch.float64)[:, None] ** powers[None, :]).to(torch.float32).to(device).contiguous()       # computed in float64, rounded once
+        self.freq = rotary_frequencies(self.rot_dims, self.rot_base)[0].to(device).contiguous() if self.rot_dims else None
+        self.dtype = dtype
+
+    def state_specs(self) -> list:
+        return [StateSpec("S", (self.heads, self.dim, self.vdim), torch.float32)]
+
+    def segments(self, sb: StepBatch) -> tuple[int, int] | None:
+        if sb.max_rows < self.SEGMENT_MIN_ROWS:
+            return None
+        chains = sb.batch * self.heads * ((self.vdim + 63) // 64)
+        segs = min(-(-self.SEGMENT_TARGET_WORKGROUPS // chains), sb.max_rows // self.SEGMENT_ROWS)
+        if segs < 2:
+            return None
+        tile = mix_ops.RETENTION_TILE
+        seg_len = -(-(-(-sb.max_rows // segs)) // tile) * tile
+        return -(-sb.max_rows // seg_len), seg_len
+
+    def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
+        p = self.inp(h)
+        if sb.decode:
+            mix_ops.retention_step(out, state["S"], p["q"], p["k"], p["v"], p["g"], self.pw, self.freq, self.interleaved, sb.tok_pos, sb.slots, self.heads, self.k_scale, self.eps)
+            return
+        o = torch.empty((sb.n, self.heads, self.vdim), dtype=torch.float32, device=h.device)
+        mix_ops.retention(o, state["S"], p["q"], p["k"], p["v"], self.pw, self.freq, self.interleaved, sb.cu, sb.slots, sb.pos0, self.k_scale, segments=self.segments(sb))
+        mix_ops.head_norm_gate(out, o, None, p["g"], mix_ops.GATE_SILU, self.eps)
+
+    def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
+        out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
+        self.attend(h, sb, state, out)
+        return F.linear(out, self.w_o)
+
+
 class ActMLP:
     KINDS = {"relu2": mix_ops.ACT_RELU2, "gelu_tanh": mix_ops.ACT_GELU_TANH, "silu": mix_ops.ACT_SILU}
 
@@ -332,7 +520,7 @@ class ActMLP:
 
 
 class GatedMLP:
-    KINDS = {"silu": mix_ops.GLU_SILU, "clamped_swish": mix_ops.GLU_CLAMPED_SWISH}
+    KINDS = {"silu": mix_ops.GLU_SILU, "clamped_swish": mix_ops.GLU_CLAMPED_SWISH, "gelu_tanh": mix_ops.GLU_GELU_TANH}
 
     def __init__(self, width: int, ff: int, act: str = "silu", limit: float = 0.0, row_gate: str | None = None):
         """row_gate: name of a [1, width] weight; the sublayer's output is multiplied by sigmoid(W_row_gate h), one number per row (applied to the hidden
@@ -346,9 +534,10 @@ class GatedMLP:
         assert self.inp.offsets["up"][1] == self.ff and self.w_down.shape == (self.width, self.ff)
         self.dtype = dtype
 
-    def hidden(self, h: torch.Tensor) -> tuple[torch.Tensor, dict]:
+    def hidden(self, h: torch.Tensor, out: torch.Tensor | None = None) -> tuple[torch.Tensor, dict]:
+        """The activation ahead of the down projection; out: where to write it (a column block of a wider matrix)."""
         p = self.inp(h)
-        a = torch.empty((h.shape[0], self.ff), dtype=self.dtype, device=h.device)
+        a = torch.empty((h.shape[0], self.ff), dtype=self.dtype, device=h.device) if out is None else out
         if self.row_gate:
             mix_ops.glu_act_rowgate(a, p["gate"], p["up"], p["row_gate"], self.kind, self.limit)
         else:
@@ -733,7 +922,6 @@ class SigmoidAttention(_SideMixer):
         self.dtype = dtype
 
     def state_specs(self) -> list:
-        from .state_cache import PagedSpec
         return [PagedSpec(self.tag + "k", (self.kv_heads * self.dim,), self.dtype), PagedSpec(self.tag + "v", (self.kv_heads * self.vdim,), self.dtype)]
 
     def run(self, p: dict, inp: FusedInput, sb: StepBatch, state: dict) -> torch.Tensor:
@@ -892,3 +1080,44 @@ class ParallelBlock:
             mix_ops.residual_norm_conv(x, y, y2, self.mult, mix_ops.RES_ADD, False, None, None, self.eps, None)
             return None
         return nxt[0].apply(x, y, y2, self.mult, mix_ops.RES_ADD, sb, nxt[1])
+
+
+class DualNormBlock:
+    """x <- x + (mixer(norm1(x)) + ff(norm2(x))), both norms RMS norms of the SAME x.  The block is entered with (h1, h2) already computed and leaves by computing the
+    next block's pair: the residual update (float32) and both norms of the next block are one kernel.  Mixer and feed-forward write into two column blocks of one
+    matrix and their output projections are one product over it, so their sum is a float32 accumulation and the stream is updated once."""
+
+    def __init__(self, width: int, eps: float, mixer, mlp):
+        self.width, self.eps, self.mixer, self.mlp = width, float(eps), mixer, mlp
+
+    def load(self, stc, prefix: str, dtype, device):
+        self.norm1 = _f32(stc, prefix + "norm1", device)
+        assert self.norm1.numel() == self.width
+        self.norm2 = None
+        self.mixer.load(stc, prefix + "mix.", dtype, device)
+        self.split = self.mixer.out_width
+        self.w_out = self.mixer.w_o
+        if self.mlp is not None:
+            self.norm2 = _f32(stc, prefix + "norm2", device)
+            self.mlp.load(stc, prefix + "mlp.", dtype, device)
+            self.w_out = torch.cat([self.mixer.w_o, self.mlp.w_down], dim=1).contiguous()
+            self.mixer.w_o, self.mlp.w_down = self.w_out[:, : self.split], self.w_out[:, self.split:]      # views: the weights are held once
+        self.dtype = dtype
+
+    def state_specs(self) -> list:
+        return self.mixer.state_specs()
+
+    def inputs(self, x: torch.Tensor, y: torch.Tensor | None, mode: int) -> tuple:
+        """x <- x | x + y, and this block's (h1, h2) (h2 None without a feed-forward)."""
+        h1 = torch.empty((x.shape[0], self.width), dtype=self.dtype, device=x.device)
+        h2 = torch.empty_like(h1) if self.mlp is not None else None
+        mix_ops.residual_norm_pair(x, y, mode, self.norm1, h1, self.norm2, h2, self.eps)
+        return h1, h2
+
+    def forward(self, h1: torch.Tensor, h2: torch.Tensor | None, sb: StepBatch, state: dict) -> torch.Tensor:
+        """What the block adds to the stream, in the activation type."""
+        cat = torch.empty((sb.n, self.w_out.shape[1]), dtype=self.dtype, device=h1.device)
+        self.mixer.attend(h1, sb, state, cat[:, : self.split])
+        if self.mlp is not None:
+            self.mlp.hidden(h2, out=cat[:, self.split:])
+        return F.linear(cat, self.w_out)

@@ -50,6 +50,7 @@ class StepBatch:
     want_rows: torch.Tensor | None = None     # int32 [m]: rows whose logits are asked for (may be empty)
     host_lens: list = field(default_factory=list)
     buffer: torch.Tensor | None = None        # the one device array that the tensors above are views of
+    shared: dict = field(default_factory=dict)         # rows that one layer of a prompt step hands to a later one
 
 
 class SlotStateCache:
