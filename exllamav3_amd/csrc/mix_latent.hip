@@ -108,7 +108,7 @@ __device__ __forceinline__ void row_trig(float* trig, int pos, const float* __re
     }
 }
 
-// One workgroup per row.  dkv (optional) [n][rank + rot_dim]: ckr[n] = [norm(latent) * kv_w | rotated key part], which also goes to the row's place in the
+// One workgroup per row and part (blockIdx.y 0: the query latent, 1: the row's own latent).  dkv (optional) [n][rank + rot_dim]: ckr[n] = [norm(latent) * kv_w | rotated key part], which also goes to the row's place in the
 // pages.  dq (optional) [n][q_rank]: cq[n] = norm(dq[n]) * q_w.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_rows_kernel(T* __restrict__ ckr, T* __restrict__ pages, const T* __restrict__ dkv, int64_t dkv_ld, const float* __restrict__ kv_w,
@@ -120,14 +120,16 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(T* __restrict__ ckr, T
     __shared__ float red[4];
     extern __shared__ float trig[];
     const int n = blockIdx.x;
-    if (dq)
+    if (blockIdx.y == 0)
     {
+        if (!dq) return;
         const T* src = dq + (int64_t) n * dq_ld;
         float ss = 0.f;
         for (int i = threadIdx.x; i < q_rank; i += 256) { const float v = to_f(src[i]); ss += v * v; }
         ss = block_sum<4>(ss, red);
         const float inv = 1.0f / sqrtf(ss / (float) q_rank + eps);
         for (int i = threadIdx.x; i < q_rank; i += 256) cq[(int64_t) n * q_rank + i] = from_f<T>(to_f(src[i]) * inv * q_w[i]);
+        return;
     }
     if (!dkv) return;
     const int pos = tok_pos[n], row = rank + rot_dim, half = rot_dims / 2;
@@ -239,7 +241,7 @@ extern "C" int exl3_mix_latent_rows(void* ckr, void* pages, const void* dkv, int
               "mix_latent_rows: bad latent");
     MIX_CHECK(rot_dims >= 0 && rot_dims <= rot_dim && rot_dims % 2 == 0 && rot_dims <= 8192, "mix_latent_rows: %d rotated dimensions of %d", rot_dims, rot_dim);
     if (n == 0) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(latent_rows_kernel<T>, dim3(n), dim3(256), (size_t) (rot_dims + 2) * sizeof(float), (hipStream_t) stream, (T*) ckr, (T*) pages, (const T*) dkv,
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(latent_rows_kernel<T>, dim3(n, dkv ? 2 : 1), dim3(256), (size_t) (rot_dims + 2) * sizeof(float), (hipStream_t) stream, (T*) ckr, (T*) pages, (const T*) dkv,
                                              dkv_ld, kv_w, (T*) cq, (const T*) dq, dq_ld, q_w, q_rank, table, table_ld, page, tok_seq, tok_pos, slots, freq, mag, interleaved, eps,
                                              rot_dim, rot_dims, rank));
     return mix_check_launch("mix_latent_rows");

@@ -173,7 +173,7 @@ __global__ __launch_bounds__(256) void heads_gate_kernel(T* __restrict__ out, in
                                                          int64_t gate_ld, int heads, int vdim)
 {
     const int n = blockIdx.x;
-    for (int t = threadIdx.x; t < heads * vdim; t += 256)
+    for (int t = blockIdx.y * 256 + threadIdx.x; t < heads * vdim; t += 256 * gridDim.y)
     {
         const int h = t / vdim, v = t - h * vdim;
         float r = to_f(a[(int64_t) n * a_row + (int64_t) h * a_head + v]);
@@ -445,7 +445,8 @@ extern "C" int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int
 {
     MIX_CHECK(out && a && n >= 0 && heads > 0 && vdim > 0 && out_ld >= (int64_t) heads * vdim && (!gate || gate_ld >= (int64_t) heads * vdim), "mix_heads_gate: bad arguments");
     if (n == 0) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(heads_gate_kernel<T>, dim3(n), dim3(256), 0, (hipStream_t) stream, (T*) out, out_ld, (const T*) a, a_row, a_head, (const T*) gate, gate_ld,
+    const int blocks = n >= 1024 ? 1 : (int) (((int64_t) heads * vdim + 255) / 256 < 64 ? ((int64_t) heads * vdim + 255) / 256 : 64);       // few rows: a row is shared out
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(heads_gate_kernel<T>, dim3(n, blocks), dim3(256), 0, (hipStream_t) stream, (T*) out, out_ld, (const T*) a, a_row, a_head, (const T*) gate, gate_ld,
                                              heads, vdim));
     return mix_check_launch("mix_heads_gate");
 }

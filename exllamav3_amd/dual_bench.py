@@ -23,11 +23,12 @@ def gated_ff(size: dict) -> int:
     return -(-size["ff"] * 2 // (3 * 128)) * 128
 
 
-def synth(size_name: str, kinds, vocab=32000, seed=0, device="cuda:0"):
-    """Random Luzinex weights and their config at a size of mixer_bench.SIZES."""
+def synth(size: dict, lt: dict, kinds, vocab=32000, seed=0, device="cuda:0", share=False):
+    """Random Luzinex weights and their config: size as in mixer_bench.SIZES, lt as in latent_bench.LATENT (q_rank: Q_RANK if it has none).  share: every
+    second latent layer reads the rows of the one before it."""
     g = torch.Generator(device=device).manual_seed(seed)
-    size, lt = SIZES[size_name], LATENT[size_name]
     w, t, layers, ff = size["width"], {}, [], gated_ff(size)
+    q_rank, lender = lt.get("q_rank", Q_RANK), None
 
     def lin(name, o, i, s=1.0):
         t[name] = (torch.randn(o, i, generator=g, device=device) * (s / math.sqrt(i))).to(torch.bfloat16)
@@ -40,9 +41,14 @@ def synth(size_name: str, kinds, vocab=32000, seed=0, device="cuda:0"):
         vec(f"l{i}.norm1", w, 1.0)
         if mix == "latent_attention":
             H, d, r, dv, rank = lt["heads"], lt["dim"], lt["rot_dim"], lt["vdim"], lt["rank"]
-            lin(p + "dq", Q_RANK, w); vec(p + "dq.norm", Q_RANK, 1.0); lin(p + "uq", H * (d + r), Q_RANK); lin(p + "dkv", rank + r, w); vec(p + "dkv.norm", rank, 1.0)
+            lin(p + "dq", q_rank, w); vec(p + "dq.norm", q_rank, 1.0); lin(p + "uq", H * (d + r), q_rank)
             lin(p + "uk", H * d, rank); lin(p + "uv", H * dv, rank)
-            mixer = {"heads": H, "dim": d, "rot_dim": r, "vdim": dv, "kv_rank": rank, "q_rank": Q_RANK, "scale": (d + r) ** -0.5, "rot": {"base": 10000.0, "dims": r}}
+            mixer = {"heads": H, "dim": d, "rot_dim": r, "vdim": dv, "kv_rank": rank, "q_rank": q_rank, "scale": (d + r) ** -0.5, "rot": {"base": 10000.0, "dims": r}}
+            if share and lender is not None:
+                mixer["kv_from"], lender = lender, None
+            else:
+                lin(p + "dkv", rank + r, w); vec(p + "dkv.norm", rank, 1.0)
+                lender = i
         elif mix == "attention":
             H, G, d = size["heads"], size["kv_heads"], size["dim"]
             dv = d
@@ -64,7 +70,7 @@ def synth(size_name: str, kinds, vocab=32000, seed=0, device="cuda:0"):
 def _make(size_name):
     def make(size, kind, reps, dev):
         from .luzinex import LuzinexModel
-        cfg, td = synth(size_name, [kind] * reps, device=dev)
+        cfg, td = synth(SIZES[size_name], LATENT[size_name], [kind] * reps, device=dev)
         return LuzinexModel(cfg, td, device=dev, dtype=torch.bfloat16)
     return make
 
