@@ -204,6 +204,34 @@ def test_one_key_stands_out_at_every_edge_of_the_window(gpu, dtype, decoded, siz
         assert (loud > 8.0) == seen, j
 
 
+@pytest.mark.parametrize("d,dv", [(64, 64), (40, 72), (64, 200), (50, 30), (96, 64), (128, 128), (104, 248), (160, 48), (192, 128), (150, 130), (144, 200), (224, 64), (256, 128), (256, 256), (201, 77)])
+@pytest.mark.parametrize("window,keep", [(1 << 30, 0), (45, 5), (200, 70)])
+def test_prompt_attention_on_the_matrix_cores_at_every_head_size(gpu, d, dv, window, keep):
+    """Every tiling of the kernel (key and value sizes, 16 or 32 rows per wave, aligned rows or not): two unequal sequences, a result in a column block, a gate per
+    value element, and scores that grow and shrink along the keys by far more than the step at which the running maximum moves."""
+    from exllamav3_amd import mix_ops
+    g = torch.Generator().manual_seed(d + dv)
+    lens, H, G, bf = [275, 37], 2, 1, torch.bfloat16
+    n = sum(lens)
+    q, k, v, gate = (torch.randn(n, w, generator=g) for w in (H * d, G * d, G * dv, H * dv))
+    ramp = torch.cat([torch.linspace(0.1, 3.0, 100), torch.linspace(3.0, 0.1, 100), torch.linspace(0.1, 6.0, n - 200)])[:, None]
+    q, k, v, gate = q.to(bf), (k * ramp).to(bf), v.to(bf), gate.to(bf)
+    sink, scale = torch.tensor([0.3, -2.0]), 1.0 / math.sqrt(d)
+    pad = 8 if (dv % 4 == 0) else 3
+    wide_out = torch.full((n, H * dv + pad), 5.0, dtype=bf, device=gpu)
+    cu, seq, pos, sl, p0, la = rows_of(gpu, lens)
+    mix_ops.attn_prefill_maps(wide_out[:, : H * dv], q.to(gpu), k.to(gpu), v.to(gpu), gate.to(gpu), sink.to(gpu), cu, seq, pos, H, G, 1, d, dv, scale, 0.0, window, mix_ops.MASK_WINDOW,
+                              max_rows=max(lens), mfma=True, keep=keep)
+    assert bool((wide_out[:, H * dv:] == 5.0).all())
+    at = 0
+    for l in lens:
+        qn, kn, vn, gn = (npy(t[at: at + l]) for t in (q, k, v, gate))
+        see = lo.kept_window(window, keep)
+        want = np.concatenate([lo.softmax_read(qn.reshape(l, H, d)[:, h], kn, vn, scale, see, float(sink[h])) for h in range(H)], axis=1) * lo.sigmoid(gn)
+        assert rel(wide_out[at: at + l, : H * dv], want) < 1.5e-2
+        at += l
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_a_sink_that_takes_most_of_the_weight(gpu, dtype):
     g = torch.Generator().manual_seed(5)
