@@ -221,7 +221,8 @@ int exl3_mix_rotate_heads(void* q, int64_t q_ld, const int32_t* tok_pos, const f
 /* The attention kernels above with: `maps` maps per head (queries [n][heads][maps][dim], keys [.][kv_heads][maps][dim]; every map of a head reads the values
  * of the head's key/value head; out [n][heads][maps][vdim]; a gate needs maps == 1), scores soft-capped to softcap tanh(score / softcap) (softcap 0: none),
  * mask EXL3_MIX_MASK_* over `window` positions, values as a column block (v_ld), and the result in float32 (out_f32) or the activation type.
- * Decode with the chunk mask reads the ring entries 0 .. (len_after - 1) % window. */
+ * Decode with the chunk mask reads the ring entries 0 .. (len_after - 1) % window.  out is a column block (row stride out_ld); the gate has gate_cols = 1 column per head
+ * or gate_cols = vdim columns per head (one per value element); keep (prompt steps, window mask): the first `keep` positions stay visible beside the window. */
 int exl3_mix_attn_prefill_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
                              const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
                              int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, int dtype, void* stream);
@@ -244,7 +245,9 @@ int exl3_mix_attn_prefill_mfma_diff(void* out, const void* q, int64_t q_ld, cons
 /* Queries and keys before the attention core, in place: per (row, head) RMS norm over dim with the weight q_norm / k_norm [dim] (NULL: none), then rotary
  * positions on the first rot_dims entries (freq [rot_dims / 2], NULL: none): pairs (i, i + rot_dims/2), or (2i, 2i+1) when `interleaved`; angle =
  * tok_pos * freq[i], cos and sin times `mag`.  q_heads and k_heads count every (head, map).  Keys and values of the rows with tok_pos >= len_after - window
- * go to ring_k [slots][window][k_heads][dim] and ring_v [slots][window][v_heads][vdim] at tok_pos % window. */
+ * go to ring_k [slots][window][k_heads][dim] and ring_v [slots][window][v_heads][vdim] at tok_pos % window.  Rotated keys are written to k_out (k itself: in
+ * place; another buffer: k stays, and v may be the same columns).  keep_first > 0: the first keep_first entries of a ring hold the sequence's first positions for good and
+ * the others go round behind them; what the newest row sees are then the first min(len_after, window) entries. */
 int exl3_mix_qk_prep(void* q, int64_t q_ld, const void* k, int64_t k_ld, void* k_out, int64_t ko_ld, const void* v, int64_t v_ld, const float* q_norm, const float* k_norm,
                      const float* freq, int rot_dims, float mag, int interleaved, float eps, void* ring_k, void* ring_v,
                      const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, const int32_t* len_after,
