@@ -236,7 +236,7 @@ def _declare(l):
 # ---- the sequence-mixer library (include/exl3_mix.h, csrc/mix_*.hip) -------------------------------------------------------------
 MIX_LIB_PATH = os.path.join(_HERE, "libexl3_mix.so")
 MIX_HEADER_PATH = os.path.join(os.path.dirname(_HERE), "include", "exl3_mix.h")
-MIX_ABI_VERSION = 5
+MIX_ABI_VERSION = 6
 _mix = None
 
 
@@ -319,7 +319,7 @@ def _declare_mix(l):
     sig("exl3_mix_act", vp, vp, i64, i32, i32, i32, i32, vp)
     sig("exl3_mix_glu_act", vp, vp, i64, vp, i64, i32, i32, i32, f32, i32, vp)
     sig("exl3_mix_token_gate", vp, vp, i64, vp, i64, i32, vp, i32, i32, i32, i32, vp)
-    sig("exl3_mix_heads_gate", vp, i64, vp, i64, i64, vp, i64, i32, i32, i32, i32, vp)
+    sig("exl3_mix_heads_gate", vp, i64, vp, i64, i64, vp, i64, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_topk_sigmoid", vp, vp, vp, vp, f32, i32, i32, i32, i32, vp)
     sig("exl3_mix_latent_prep", vp, vp, vp, i64, vp, vp, i64, vp, vp, vp, vp, vp, f32, f32, i32, i32, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_latent_fill_k", vp, i64, vp, i32, i32, i32, i32, i32, i32, vp)
@@ -328,9 +328,9 @@ def _declare_mix(l):
     sig("exl3_mix_latent_rows", vp, vp, vp, i64, vp, vp, vp, i64, vp, i32, vp, i64, i32, vp, vp, vp, vp, f32, i32, f32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_rotate_heads", vp, i64, vp, vp, f32, i32, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_latent_decode", vp, i64, i64, vp, i64, i64, vp, i64, vp, vp, vp, vp, vp, i64, i32, i32, i32, i32, i32, i32, f32, i32, i32, vp)
-    sig("exl3_mix_attn_prefill_ex", vp, i64, i32, vp, i64, vp, i64, vp, i64, vp, i64, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, i32, vp)
-    sig("exl3_mix_attn_prefill_mfma_ex", vp, i64, i32, vp, i64, vp, i64, vp, i64, vp, i64, i32, vp, vp, i32, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, vp)
-    sig("exl3_mix_attn_decode_ex", vp, i64, i32, vp, i64, vp, vp, vp, i64, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, vp)
+    sig("exl3_mix_attn_prefill_ex", vp, i64, i32, vp, i64, vp, i64, vp, i64, vp, i64, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, f32, i32, vp)
+    sig("exl3_mix_attn_prefill_mfma_ex", vp, i64, i32, vp, i64, vp, i64, vp, i64, vp, i64, i32, vp, vp, i32, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, i32, f32, vp)
+    sig("exl3_mix_attn_decode_ex", vp, i64, i32, vp, i64, vp, vp, vp, i64, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, f32, i32, i32, f32, i32, vp)
     sig("exl3_mix_qk_prep", vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, i32, f32, i32, f32, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_diff_combine", vp, vp, f32, f32, f32, vp, i64, i32, i32, i32, i32, vp)
     sig("exl3_mix_residual_rms", vp, vp, i64, i32, vp, f32, vp, i64, vp, i32, vp, vp, vp, vp, i32, i32, i32, vp)
@@ -358,4 +358,10 @@ def _declare_mix(l):
     sig("exl3_mix_retention", vp, vp, vp, i64, vp, i64, vp, i64, vp, i32, vp, i32, i32, vp, vp, vp, i32, i32, i32, i32, f32, i32, i32, vp, i32, vp)
     sig("exl3_mix_retention_step", vp, i64, vp, vp, i64, vp, i64, vp, i64, vp, i64, vp, i32, vp, i32, i32, vp, vp, i32, i32, i32, i32, f32, f32, i32, vp)
     sig("exl3_mix_head_norm_gate", vp, i64, vp, vp, i32, vp, i64, i32, f32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_embed_norm", vp, vp, i64, vp, vp, vp, f32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_conv_prep", vp, vp, i64, vp, i32, vp, vp, vp, vp, i32, f32, i32, f32, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_token_shift", vp, vp, i64, vp, vp, i32, vp, vp, vp, vp, vp, i32, i32, i32, vp)
+    sig("exl3_mix_decay_log", vp, vp, i64, vp, vp, i32, i32, i32, i32, vp)
+    sig("exl3_mix_timemix", vp, vp, i64, vp, i64, vp, f32, vp, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp, vp, i32, vp)
+    sig("exl3_mix_timemix_step", vp, i64, vp, vp, i64, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, vp)
     sig("exl3_mix_rms_pair", vp, vp, i64, vp, vp, i64, vp, f32, f32, i32, i32, i32, vp)

@@ -44,7 +44,7 @@ template <typename T, int MAXV, typename TO, int NW>
 __global__ __launch_bounds__(64 * NW) void attn_prefill_kernel(TO* __restrict__ out, int64_t out_ld, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ k, int64_t k_ld,
                                                           const T* __restrict__ v, int64_t v_ld, const T* __restrict__ gate, int64_t gate_ld, int gate_cols, const float* __restrict__ sink,
                                                           const int32_t* __restrict__ cu, const int32_t* __restrict__ tok_seq, const int32_t* __restrict__ tok_pos,
-                                                          int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep)
+                                                          int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, float out_scale)
 {
     extern __shared__ float smem[];
     const int n = blockIdx.x, h = blockIdx.y;                 // h counts (head, map)
@@ -53,7 +53,7 @@ __global__ __launch_bounds__(64 * NW) void attn_prefill_kernel(TO* __restrict__ 
     const int i = n - first;                                  // the row's place in its sequence == its position (the sequence starts in this step)
     const int lo = mask == EXL3_MIX_MASK_CHUNK ? (i / window) * window : max(0, i - window + 1);
     const bool by_head = gate && gate_cols == 1;
-    const float gt = by_head ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) : 1.0f;
+    const float gt = by_head ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) * out_scale : out_scale;
     const T* grow = gate && !by_head ? gate + (int64_t) n * gate_ld + (int64_t) h * vdim : nullptr;
     if (keep > 0)                                             // keys 0 .. keep - 1, then lo .. i
     {
@@ -76,7 +76,7 @@ template <typename T, int MAXV, typename TO, int NW>
 __global__ __launch_bounds__(64 * NW) void attn_decode_kernel(TO* __restrict__ out, int64_t out_ld, const T* __restrict__ q, int64_t q_ld, const T* __restrict__ ring_k,
                                                          const T* __restrict__ ring_v, const T* __restrict__ gate, int64_t gate_ld, int gate_cols, const float* __restrict__ sink,
                                                          const int32_t* __restrict__ slots, const int32_t* __restrict__ len_after,
-                                                         int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask)
+                                                         int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, float out_scale)
 {
     extern __shared__ float smem[];
     const int n = blockIdx.x, h = blockIdx.y;
@@ -85,7 +85,7 @@ __global__ __launch_bounds__(64 * NW) void attn_decode_kernel(TO* __restrict__ o
     const int count = mask == EXL3_MIX_MASK_CHUNK ? (len - 1) % window + 1 : min(len, window);
     const int64_t row0 = (int64_t) slots[n] * window;
     const bool by_head = gate && gate_cols == 1;
-    const float gt = by_head ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) : 1.0f;
+    const float gt = by_head ? sigmoid_f(to_f(gate[(int64_t) n * gate_ld + h])) * out_scale : out_scale;
     const T* grow = gate && !by_head ? gate + (int64_t) n * gate_ld + (int64_t) h * vdim : nullptr;
     const T* kb = ring_k + (row0 * kheads + kh) * dim;
     attn_row<T, MAXV, TO, NW>(out + (int64_t) n * out_ld + (int64_t) h * vdim, q + (int64_t) n * q_ld + (int64_t) h * dim, q, dim,
@@ -139,7 +139,7 @@ static int attn_check(const char* what, int n, int heads, int kv_heads, int maps
 
 extern "C" int exl3_mix_attn_prefill_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
                                         const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
-                                        int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, int dtype, void* stream)
+                                        int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, float out_scale, int dtype, void* stream)
 {
     MIX_CHECK(out && q && k && v && cu && tok_seq && tok_pos, "mix_attn_prefill: null pointer");
     if (int rc = attn_check("mix_attn_prefill", n, heads, kv_heads, maps, dim, vdim, window, mask, softcap, gate, gate_cols, gate_ld, out_ld)) return rc;
@@ -149,7 +149,7 @@ extern "C" int exl3_mix_attn_prefill_ex(void* out, int64_t out_ld, int out_f32, 
     if (n == 0) return EXL3_MIX_OK;
     const bool wide = false;
     ATTN_LAUNCH(attn_prefill_kernel, out_ld, (const T*) q, q_ld, (const T*) k, k_ld, (const T*) v, v_ld, (const T*) gate, gate_ld, gate_cols, sink, cu, tok_seq, tok_pos,
-                heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep);
+                heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, out_scale);
     return mix_check_launch("mix_attn_prefill");
 }
 
@@ -158,12 +158,12 @@ extern "C" int exl3_mix_attn_prefill(void* out, const void* q, int64_t q_ld, con
                                      int n, int heads, int kv_heads, int dim, int vdim, float scale, int window, int dtype, void* stream)
 {
     return exl3_mix_attn_prefill_ex(out, (int64_t) heads * vdim, 0, q, q_ld, k, k_ld, v_norm, (int64_t) kv_heads * vdim, gate, gate_ld, 1, sink, cu, tok_seq, tok_pos, n, heads, kv_heads, 1, dim, vdim,
-                                    scale, 0.f, window, EXL3_MIX_MASK_WINDOW, 0, dtype, stream);
+                                    scale, 0.f, window, EXL3_MIX_MASK_WINDOW, 0, 1.0f, dtype, stream);
 }
 
 extern "C" int exl3_mix_attn_decode_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* ring_k, const void* ring_v,
                                        const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* slots, const int32_t* len_after,
-                                       int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int dtype, void* stream)
+                                       int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, float out_scale, int dtype, void* stream)
 {
     MIX_CHECK(out && q && ring_k && ring_v && slots && len_after, "mix_attn_decode: null pointer");
     if (int rc = attn_check("mix_attn_decode", n, heads, kv_heads, maps, dim, vdim, window, mask, softcap, gate, gate_cols, gate_ld, out_ld)) return rc;
@@ -171,7 +171,7 @@ extern "C" int exl3_mix_attn_decode_ex(void* out, int64_t out_ld, int out_f32, c
     if (n == 0) return EXL3_MIX_OK;
     const bool wide = (int64_t) n * heads * maps <= 256 && window > 256 && vdim <= 256;
     ATTN_LAUNCH(attn_decode_kernel, out_ld, (const T*) q, q_ld, (const T*) ring_k, (const T*) ring_v, (const T*) gate, gate_ld, gate_cols, sink, slots, len_after,
-                heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask);
+                heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, out_scale);
     return mix_check_launch("mix_attn_decode");
 }
 
@@ -180,5 +180,5 @@ extern "C" int exl3_mix_attn_decode(void* out, const void* q, int64_t q_ld, cons
                                     int n, int heads, int kv_heads, int dim, int vdim, float scale, int window, int dtype, void* stream)
 {
     return exl3_mix_attn_decode_ex(out, (int64_t) heads * vdim, 0, q, q_ld, ring_k, ring_v, gate, gate_ld, 1, sink, slots, len_after, n, heads, kv_heads, 1, dim, vdim, scale, 0.f, window,
-                                   EXL3_MIX_MASK_WINDOW, dtype, stream);
+                                   EXL3_MIX_MASK_WINDOW, 1.0f, dtype, stream);
 }

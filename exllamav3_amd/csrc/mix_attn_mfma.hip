@@ -23,7 +23,8 @@
 // sliding window -- both give every row a first visible key lo(i) that never decreases with i, which is all the tile logic uses; a soft cap on the
 // scores, cap tanh(score / cap), applied to the scaled scores before the running maximum (tanh is increasing, so the largest raw score still is the
 // largest score); a float32 result; the first `keep` positions visible to every row beside its window (the tiles that hold them are visited first, then
-// those of the window: a row's mask is "in the window, or among the first"); and an output gate per head or per value element, applied in the epilogue.
+// those of the window: a row's mask is "in the window, or among the first"); and an output gate per head or per value element and a factor on the
+// result, applied in the epilogue.
 #include "mix_common.cuh"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -63,7 +64,7 @@ void attn_prefill_mfma_kernel(void* __restrict__ out_any, int64_t out_ld, int ou
                               int64_t k_ld, const bf16_t* __restrict__ v, int64_t v_ld, const bf16_t* __restrict__ gate, int64_t gate_ld, int gate_cols,
                               const float* __restrict__ sink, const int32_t* __restrict__ cu,
                               int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep,
-                              int o_vec)
+                              float out_scale, int o_vec)
 {
     constexpr int NT = 64 * AM_ROWS / (16 * QG), DP = KD * 32, KS = DP + AM_KPAD, VS = NV * 16 + AM_VPAD, NS = AM_KEYS / 16;
     constexpr int KC = DP / 8, VC = NV * 2;                       // 16-byte chunks per key
@@ -277,7 +278,7 @@ void attn_prefill_mfma_kernel(void* __restrict__ out_any, int64_t out_ld, int ou
         if (qi[u] >= len) continue;
         const int64_t n = first + qi[u];
         const bool by_head = gate && gate_cols == 1;
-        const float gt = by_head ? sigmoid_f(to_f(gate[n * gate_ld + h])) : 1.0f;
+        const float gt = by_head ? sigmoid_f(to_f(gate[n * gate_ld + h])) * out_scale : out_scale;
         const bf16_t* grow = gate && !by_head ? gate + n * gate_ld + (int64_t) h * vdim : nullptr;
         const float f = (l[u] > 0.f ? 1.0f / l[u] : 0.f) * gt;
         const int64_t o0 = n * out_ld + (int64_t) h * vdim;
@@ -323,13 +324,13 @@ extern "C" int exl3_mix_attn_prefill_mfma(void* out, const void* q, int64_t q_ld
                                           int batch, int max_rows, int heads, int kv_heads, int dim, int vdim, float scale, int window, void* stream)
 {
     return exl3_mix_attn_prefill_mfma_ex(out, (int64_t) heads * vdim, 0, q, q_ld, k, k_ld, v_norm, (int64_t) kv_heads * vdim, gate, gate_ld, 1, sink, cu, batch, max_rows, heads, kv_heads, 1, dim, vdim,
-                                         scale, 0.f, window, EXL3_MIX_MASK_WINDOW, 0, stream);
+                                         scale, 0.f, window, EXL3_MIX_MASK_WINDOW, 0, 1.0f, stream);
 }
 
 extern "C" int exl3_mix_attn_prefill_mfma_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v_norm, int64_t v_ld,
                                              const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu,
                                              int batch, int max_rows, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep,
-                                             void* stream)
+                                             float out_scale, void* stream)
 {
     MIX_CHECK(out && q && k && v_norm && cu, "mix_attn_prefill_mfma: null pointer");
     MIX_CHECK(batch >= 0 && max_rows >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && maps >= 1 && heads * maps <= 65535 && batch <= 65535,
@@ -350,7 +351,7 @@ extern "C" int exl3_mix_attn_prefill_mfma_ex(void* out, int64_t out_ld, int out_
     #define AM_LAUNCH_C(KDV, NVV, KTV, QGV, CAPV, VECV) \
         hipLaunchKernelGGL((attn_prefill_mfma_kernel<KDV, NVV, KTV, QGV, CAPV, VECV>), grid, dim3(64 * AM_ROWS / (16 * QGV)), AM_LDS(KDV, NVV, KTV), (hipStream_t) stream, out, out_ld, out_f32, \
                            (const bf16_t*) q, q_ld, (const bf16_t*) k, k_ld, (const bf16_t*) v_norm, v_ld, (const bf16_t*) gate, gate_ld, gate_cols, sink, cu, heads, kv_heads, maps, dim, vdim, \
-                           scale, softcap, window, mask, keep, o_vec)
+                           scale, softcap, window, mask, keep, out_scale, o_vec)
     #define AM_LAUNCH(KDV, NVV, KTV, QGV) do { \
         static_assert(AM_LDS(KDV, NVV, KTV) <= 65536, "tile does not fit the LDS"); \
         if (vec) { if (softcap > 0.f) AM_LAUNCH_C(KDV, NVV, KTV, QGV, true, true); else AM_LAUNCH_C(KDV, NVV, KTV, QGV, false, true); } \

@@ -87,6 +87,46 @@ __device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.f) -
 // log(1 + exp(z)) without overflow
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
+// Rings of `rows` entries of which the first `keep` belong to the first `keep` positions: where position pos lives, and whether a step that brings its sequence
+// to `len` positions leaves it there.  A sequence's visible entries are always the first min(len, rows).
+__device__ __forceinline__ int ring_entry(int pos, int rows, int keep) { return pos < keep ? pos : keep + (pos - keep) % (rows - keep); }
+__device__ __forceinline__ bool ring_holds(int pos, int len, int rows, int keep) { return pos < keep || pos >= len - (rows - keep); }
+
+// V consecutive elements at once, as one access of 8 or 16 bytes where V of them are that many (p aligned to it), else one by one
+template <int B> struct raw_bytes;
+template <> struct raw_bytes<8> { typedef uint2 type; };
+template <> struct raw_bytes<16> { typedef uint4 type; };
+template <typename T, int V> __device__ __forceinline__ void load_n(const T* p, float (&o)[V])
+{
+    if constexpr (V * sizeof(T) == 8 || V * sizeof(T) == 16)
+    {
+        union { typename raw_bytes<V * sizeof(T)>::type v; T e[V]; } t;
+        t.v = *(const typename raw_bytes<V * sizeof(T)>::type*) p;
+        #pragma unroll
+        for (int e = 0; e < V; ++e) o[e] = to_f(t.e[e]);
+    }
+    else
+    {
+        #pragma unroll
+        for (int e = 0; e < V; ++e) o[e] = to_f(p[e]);
+    }
+}
+template <typename T, int V> __device__ __forceinline__ void store_n(T* p, const float (&o)[V])
+{
+    if constexpr (V * sizeof(T) == 8 || V * sizeof(T) == 16)
+    {
+        union { typename raw_bytes<V * sizeof(T)>::type v; T e[V]; } t;
+        #pragma unroll
+        for (int e = 0; e < V; ++e) t.e[e] = from_f<T>(o[e]);
+        *(typename raw_bytes<V * sizeof(T)>::type*) p = t.v;
+    }
+    else
+    {
+        #pragma unroll
+        for (int e = 0; e < V; ++e) p[e] = from_f<T>(o[e]);
+    }
+}
+
 // error reporting shared by the translation units of this library (thread-local message, negative return codes)
 void mix_set_error(const char* fmt, ...);
 int  mix_check_launch(const char* what);

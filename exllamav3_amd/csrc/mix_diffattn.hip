@@ -9,11 +9,6 @@
 // Sums of squares, angles, cos / sin and the combination are float32.
 #include "mix_common.cuh"
 
-// Rings of `rows` entries of which the first `keep` belong to the first `keep` positions: where position pos lives, and whether a step that brings its sequence
-// to `len` positions leaves it there.  A sequence's visible entries are always the first min(len, rows).
-__device__ __forceinline__ int ring_entry(int pos, int rows, int keep) { return pos < keep ? pos : keep + (pos - keep) % (rows - keep); }
-__device__ __forceinline__ bool ring_holds(int pos, int len, int rows, int keep) { return pos < keep || pos >= len - (rows - keep); }
-
 // One workgroup of QP_WAVES waves per row: cos / sin of the row's position are computed once into LDS, then the waves take the row's items -- q_heads
 // query vectors, k_heads key vectors, v_heads value vectors -- in turn.  q [n][q_heads][dim], k [n][k_heads][dim], v [n][v_heads][vdim] are column blocks
 // of wider matrices (row strides); q_heads and k_heads count (head, map).  ring_k [slots][window][k_heads][dim], ring_v [slots][window][v_heads][vdim],

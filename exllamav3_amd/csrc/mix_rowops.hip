@@ -24,6 +24,28 @@ __global__ __launch_bounds__(ROW_THREADS) void embed_copy_kernel(float* __restri
     }
 }
 
+// x[n] = table row of tokens[n] over its root mean square, times w; xc (optional): the same in the activation type
+template <typename T>
+__global__ __launch_bounds__(ROW_THREADS) void embed_norm_kernel(float* __restrict__ x, T* __restrict__ xc, int64_t xc_ld, const T* __restrict__ table,
+                                                                 const int32_t* __restrict__ tokens, const float* __restrict__ w, float eps, int width, int vocab)
+{
+    __shared__ float red[ROW_WAVES];
+    const int n = blockIdx.x;
+    int tok = tokens[n];
+    tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
+    const T* src = table + (int64_t) tok * width;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < width; i += ROW_THREADS) { const float v = to_f(src[i]); ss += v * v; }
+    ss = block_sum<ROW_WAVES>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float) width + eps);
+    for (int i = threadIdx.x; i < width; i += ROW_THREADS)
+    {
+        const float v = to_f(src[i]) * inv * w[i];
+        x[(int64_t) n * width + i] = v;
+        if (xc) xc[(int64_t) n * xc_ld + i] = from_f<T>(v);
+    }
+}
+
 // x[n] = table[tokens[n]] * scale + P(tok_pos[n]): a sinusoidal position vector, entry 2i = sin(p f_i), entry 2i + 1 = cos(p f_i), f_i = freq[i] (float32;
 // the angle is the float32 product of the position and the frequency)
 template <typename T>
@@ -62,8 +84,10 @@ __global__ __launch_bounds__(ROW_THREADS) void layer_norm_rows_kernel(T* __restr
 }
 
 // mode 0: x stays; 1: x += y'; 2: x = y'   with y' = y, or y / rms(y) * rms_w when rms_w is given.
-// out 0: nothing; 1: h = x in the activation type; 2: h = tanh(alpha x) w + b.
-template <typename T>
+// out 0: nothing; 1: h = x in the activation type; 2: h = tanh(alpha x) w + b.  V: elements per thread and access (4 when the rows allow it); a thread keeps its
+// first RN_HELD pieces of y in registers between the sum of squares and the update, later ones are read again.
+#define RN_HELD 4
+template <typename T, int V>
 __global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(float* __restrict__ x, const T* __restrict__ y, int64_t y_ld, int mode, const float* __restrict__ rms_w,
                                                                     float eps, int out, float alpha, const float* __restrict__ w, const float* __restrict__ b,
                                                                     T* __restrict__ h, int64_t h_ld, int width)
@@ -72,27 +96,77 @@ __global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(float* __res
     const int n = blockIdx.x;
     float* xr = x + (int64_t) n * width;
     const T* yr = y + (int64_t) n * y_ld;
+    T* hr = h + (int64_t) n * h_ld;
+    float held[RN_HELD][V], xv[RN_HELD][V];
+    #pragma unroll
+    for (int u = 0; u < RN_HELD; ++u)                                  // all loads of the held pieces are in flight before the first sum
+    {
+        const int i = (u * ROW_THREADS + threadIdx.x) * V;
+        #pragma unroll
+        for (int e = 0; e < V; ++e) { held[u][e] = 0.f; xv[u][e] = 0.f; }
+        if (i >= width) continue;
+        if (mode != 0) load_n<T, V>(yr + i, held[u]);
+        if (mode != 2) load_n<float, V>(xr + i, xv[u]);
+    }
     float inv = 1.0f;
     if (mode != 0 && rms_w)
     {
         float ss = 0.f;
-        for (int i = threadIdx.x; i < width; i += ROW_THREADS) { const float v = to_f(yr[i]); ss += v * v; }
+        #pragma unroll
+        for (int u = 0; u < RN_HELD; ++u)
+        {
+            #pragma unroll
+            for (int e = 0; e < V; ++e) ss += held[u][e] * held[u][e];
+        }
+        for (int i = (RN_HELD * ROW_THREADS + threadIdx.x) * V; i < width; i += ROW_THREADS * V)
+        {
+            float t[V];
+            load_n<T, V>(yr + i, t);
+            #pragma unroll
+            for (int e = 0; e < V; ++e) ss += t[e] * t[e];
+        }
         ss = block_sum<ROW_WAVES>(ss, red);
         inv = 1.0f / sqrtf(ss / (float) width + eps);
     }
-    T* hr = h + (int64_t) n * h_ld;
-    for (int i = threadIdx.x; i < width; i += ROW_THREADS)
+    auto update = [&](int i, float (&a)[V], float (&v)[V]) __attribute__((always_inline))
     {
-        float v = xr[i];
+        float t[V];
         if (mode != 0)
         {
-            float a = to_f(yr[i]);
-            if (rms_w) a = a * inv * rms_w[i];
-            v = mode == 1 ? v + a : a;
-            xr[i] = v;
+            if (rms_w)
+            {
+                load_n<float, V>(rms_w + i, t);
+                #pragma unroll
+                for (int e = 0; e < V; ++e) a[e] = a[e] * inv * t[e];
+            }
+            #pragma unroll
+            for (int e = 0; e < V; ++e) v[e] = mode == 1 ? v[e] + a[e] : a[e];
+            store_n<float, V>(xr + i, v);
         }
-        if (out == 1) hr[i] = from_f<T>(v);
-        else if (out == 2) hr[i] = from_f<T>(tanhf(alpha * v) * w[i] + b[i]);
+        if (out == 1) store_n<T, V>(hr + i, v);
+        else if (out == 2)
+        {
+            float wv[V], bv[V];
+            load_n<float, V>(w + i, wv); load_n<float, V>(b + i, bv);
+            #pragma unroll
+            for (int e = 0; e < V; ++e) t[e] = tanhf(alpha * v[e]) * wv[e] + bv[e];
+            store_n<T, V>(hr + i, t);
+        }
+    };
+    #pragma unroll
+    for (int u = 0; u < RN_HELD; ++u)
+    {
+        const int i = (u * ROW_THREADS + threadIdx.x) * V;
+        if (i < width) update(i, held[u], xv[u]);
+    }
+    for (int i = (RN_HELD * ROW_THREADS + threadIdx.x) * V; i < width; i += ROW_THREADS * V)
+    {
+        float a[V], v[V];
+        #pragma unroll
+        for (int e = 0; e < V; ++e) { a[e] = 0.f; v[e] = 0.f; }
+        if (mode != 0) load_n<T, V>(yr + i, a);
+        if (mode != 2) load_n<float, V>(xr + i, v);
+        update(i, a, v);
     }
 }
 
@@ -167,17 +241,17 @@ __global__ __launch_bounds__(64) void token_gate_kernel(T* __restrict__ out, con
         out[(int64_t) n * dim + j] = from_f<T>(gelu_tanh_f(to_f(gate[(int64_t) n * gate_ld + j])) * to_f(e[j]));
 }
 
-// out[n][h * vdim + v] = a[n * a_row + h * a_head + v] * (gate ? sigmoid(gate[n][h * vdim + v]) : 1)
+// out[n][h * vdim + v] = a[n * a_row + h * a_head + v] * (gate ? sigmoid(gate[n][h * vdim + v]) : 1); by_head: sigmoid(gate[n][h])
 template <typename T>
 __global__ __launch_bounds__(256) void heads_gate_kernel(T* __restrict__ out, int64_t out_ld, const T* __restrict__ a, int64_t a_row, int64_t a_head, const T* __restrict__ gate,
-                                                         int64_t gate_ld, int heads, int vdim)
+                                                         int64_t gate_ld, int by_head, int heads, int vdim)
 {
     const int n = blockIdx.x;
     for (int t = blockIdx.y * 256 + threadIdx.x; t < heads * vdim; t += 256 * gridDim.y)
     {
         const int h = t / vdim, v = t - h * vdim;
         float r = to_f(a[(int64_t) n * a_row + (int64_t) h * a_head + v]);
-        if (gate) r *= sigmoid_f(to_f(gate[(int64_t) n * gate_ld + t]));
+        if (gate) r *= sigmoid_f(to_f(gate[(int64_t) n * gate_ld + (by_head ? h : t)]));
         out[(int64_t) n * out_ld + t] = from_f<T>(r);
     }
 }
@@ -366,6 +440,14 @@ extern "C" int exl3_mix_embed_copy(float* x, void* xc, int64_t xc_ld, const void
     return mix_check_launch("mix_embed_copy");
 }
 
+extern "C" int exl3_mix_embed_norm(float* x, void* xc, int64_t xc_ld, const void* table, const int32_t* tokens, const float* w, float eps, int n, int width, int vocab, int dtype, void* stream)
+{
+    MIX_CHECK(x && table && tokens && w && n >= 0 && width > 0 && vocab > 0 && (!xc || xc_ld >= width), "mix_embed_norm: bad arguments");
+    if (n == 0) return EXL3_MIX_OK;
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(embed_norm_kernel<T>, dim3(n), dim3(ROW_THREADS), 0, (hipStream_t) stream, x, (T*) xc, xc_ld, (const T*) table, tokens, w, eps, width, vocab));
+    return mix_check_launch("mix_embed_norm");
+}
+
 extern "C" int exl3_mix_residual_norm(float* x, const void* y, int64_t y_ld, int mode, const float* rms_w, float eps, int out, float alpha, const float* w, const float* b,
                                       void* h, int64_t h_ld, int n, int width, int dtype, void* stream)
 {
@@ -374,8 +456,12 @@ extern "C" int exl3_mix_residual_norm(float* x, const void* y, int64_t y_ld, int
     MIX_CHECK(out == 0 || (h && h_ld >= width), "mix_residual_norm: an output is needed");
     MIX_CHECK(out != 2 || (w && b), "mix_residual_norm: the norm needs its weight and bias");
     if (n == 0 || (mode == 0 && out == 0)) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(residual_norm_kernel<T>, dim3(n), dim3(ROW_THREADS), 0, (hipStream_t) stream, x, (const T*) y, y_ld, mode, rms_w, eps, out, alpha,
-                                             w, b, (T*) h, h_ld, width));
+    const bool by4 = width % 4 == 0 && (uintptr_t) x % 16 == 0 && (mode == 0 || (y_ld % 4 == 0 && (uintptr_t) y % 16 == 0)) && (out == 0 || (h_ld % 4 == 0 && (uintptr_t) h % 16 == 0)) &&
+                     (uintptr_t) rms_w % 16 == 0 && (uintptr_t) w % 16 == 0 && (uintptr_t) b % 16 == 0;
+    #define RN_LAUNCH(VV) hipLaunchKernelGGL((residual_norm_kernel<T, VV>), dim3(n), dim3(ROW_THREADS), 0, (hipStream_t) stream, x, (const T*) y, y_ld, mode, rms_w, eps, out, alpha, w, b, \
+                                             (T*) h, h_ld, width)
+    MIX_DISPATCH_T(dtype, if (by4) RN_LAUNCH(4); else RN_LAUNCH(1));
+    #undef RN_LAUNCH
     return mix_check_launch("mix_residual_norm");
 }
 
@@ -441,13 +527,14 @@ extern "C" int exl3_mix_token_gate(void* out, const void* gate, int64_t gate_ld,
     return mix_check_launch("mix_token_gate");
 }
 
-extern "C" int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int n, int heads, int vdim, int dtype, void* stream)
+extern "C" int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int gate_cols, int n, int heads, int vdim, int dtype, void* stream)
 {
-    MIX_CHECK(out && a && n >= 0 && heads > 0 && vdim > 0 && out_ld >= (int64_t) heads * vdim && (!gate || gate_ld >= (int64_t) heads * vdim), "mix_heads_gate: bad arguments");
+    MIX_CHECK(out && a && n >= 0 && heads > 0 && vdim > 0 && out_ld >= (int64_t) heads * vdim && (!gate || ((gate_cols == 1 || gate_cols == vdim) && gate_ld >= (int64_t) heads * gate_cols)),
+              "mix_heads_gate: bad arguments (a gate has 1 or vdim columns per head)");
     if (n == 0) return EXL3_MIX_OK;
     const int blocks = n >= 1024 ? 1 : (int) (((int64_t) heads * vdim + 255) / 256 < 64 ? ((int64_t) heads * vdim + 255) / 256 : 64);       // few rows: a row is shared out
     MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(heads_gate_kernel<T>, dim3(n, blocks), dim3(256), 0, (hipStream_t) stream, (T*) out, out_ld, (const T*) a, a_row, a_head, (const T*) gate, gate_ld,
-                                             heads, vdim));
+                                             gate_cols == 1, heads, vdim));
     return mix_check_launch("mix_heads_gate");
 }
 

@@ -264,6 +264,17 @@ def embed_copy(x: torch.Tensor, xc_view: torch.Tensor | None, table: torch.Tenso
                                               code(table.dtype), _stream(x)))
 
 
+def embed_norm(x: torch.Tensor, xc_view: torch.Tensor | None, table: torch.Tensor, tokens: torch.Tensor, w: torch.Tensor, eps: float):
+    """x (float32) = RMS norm of the tokens' table rows with weight w; xc_view: the same in the activation type."""
+    n, width = x.shape
+    _f32c(x, "x"); _f32c(w, "w"); _i32c(tokens, "tokens")
+    _req(tokens.numel() == n and table.is_contiguous() and table.shape[1] == width == w.numel(), "embed_norm: shapes")
+    if xc_view is not None:
+        _req(xc_view.dtype == table.dtype and xc_view.shape[0] == n, "embed_norm: the copy has the table's element type")
+    _check(_lib.mixlib().exl3_mix_embed_norm(_p(x), _p(xc_view), 0 if xc_view is None else _view(xc_view, width, "xc"), _p(table), _p(tokens), _p(w), eps, n, width, table.shape[0],
+                                              code(table.dtype), _stream(x)))
+
+
 def residual_norm(x: torch.Tensor, y_view: torch.Tensor | None, mode: int, rms_w: torch.Tensor | None, eps: float, out: int, alpha: float, w: torch.Tensor | None,
                   b: torch.Tensor | None, h_view: torch.Tensor | None):
     """x (float32 residual, in place) = x | x + y' | y', y' = y or y / rms(y) * rms_w; h = nothing | x in the activation type | tanh(alpha x) w + b."""
@@ -316,12 +327,11 @@ def token_gate(out: torch.Tensor, gate_view: torch.Tensor, table: torch.Tensor, 
 
 
 def heads_gate(out: torch.Tensor, a: torch.Tensor, a_row: int, a_head: int, gate_view: torch.Tensor | None, heads: int, vdim: int):
-    """a is addressed as base + n * a_row + h * a_head + v (token-major or head-major); the gate, if any, is [n, heads * vdim] before its sigmoid."""
+    """a is addressed as base + n * a_row + h * a_head + v (token-major or head-major); the gate, if any, is [n, heads * vdim] or [n, heads] before its sigmoid."""
     n = out.shape[0]
     _req(a.dtype == out.dtype and a.numel() >= n * heads * vdim, "heads_gate: shapes")
-    if gate_view is not None:
-        _req(gate_view.dtype == out.dtype and gate_view.shape[0] == n, "heads_gate: gate")
-    _check(_lib.mixlib().exl3_mix_heads_gate(_p(out), _view(out, heads * vdim, "out"), _p(a), a_row, a_head, _p(gate_view), 0 if gate_view is None else _view(gate_view, heads * vdim, "gate"), n, heads, vdim,
+    gate, gate_ld, gate_cols = _gate_args(gate_view, n, heads, vdim, out.dtype, "heads_gate")
+    _check(_lib.mixlib().exl3_mix_heads_gate(_p(out), _view(out, heads * vdim, "out"), _p(a), a_row, a_head, gate, gate_ld, gate_cols, n, heads, vdim,
                                               code(out.dtype), _stream(out)))
 
 
@@ -482,6 +492,31 @@ def qk_prep(q_view, k_view, v_view, q_norm, k_norm, freq, mag: float, interleave
                                            n, q_heads, k_heads, v_heads, dim, vdim, window, keep_first, code(q_view.dtype), _stream(q_view)))
 
 
+def conv_prep(out, x_view, conv_w, conv_ring, q_norm, k_norm, freq, mag: float, interleaved: bool, eps: float, ring_k, ring_v, sb, q_heads: int, keep_first: int = 0):
+    """qk_prep for projections q | k | v (x_view [n, C]) that pass a short causal convolution first: conv_w [taps, C] float32, conv_ring [slots, max(taps - 1, 1), C] the
+    last projected rows of every slot; out [n, C] receives normed and rotated queries and keys and the convolved values.  sb: the step's StepBatch (or any object with its
+    tok_seq, tok_pos, slots, pos0, len_after)."""
+    n, C = x_view.shape
+    n_slots, rows, kv_heads, dim = ring_k.shape
+    vdim, taps = ring_v.shape[3], conv_w.shape[0]
+    _f32c(conv_w, "conv_w")
+    _req(C == q_heads * dim + kv_heads * (dim + vdim) and out.shape == (n, C) and out.is_contiguous() and conv_w.shape[1] == C, "conv_prep: step shapes")
+    _req(ring_v.shape[:3] == (n_slots, rows, kv_heads) and ring_k.is_contiguous() and ring_v.is_contiguous() and conv_ring.is_contiguous()
+         and conv_ring.shape == (n_slots, max(taps - 1, 1), C), "conv_prep: ring shapes")
+    _req(out.dtype == x_view.dtype == conv_ring.dtype == ring_k.dtype == ring_v.dtype, "conv_prep: element types")
+    for t, nm in ((sb.tok_seq, "tok_seq"), (sb.tok_pos, "tok_pos"), (sb.slots, "slots"), (sb.pos0, "pos0"), (sb.len_after, "len_after")):
+        _i32c(t, nm)
+    for t, nm in ((q_norm, "q_norm"), (k_norm, "k_norm")):
+        if t is not None:
+            _f32c(t, nm); _req(t.numel() == dim, f"conv_prep: {nm}")
+    if freq is not None:
+        _f32c(freq, "freq")
+    _req(sb.tok_seq.numel() == n and sb.tok_pos.numel() == n, "conv_prep: rows")
+    _check(_lib.mixlib().exl3_mix_conv_prep(_p(out), _p(x_view), _view(x_view, C, "x"), _p(conv_w), taps, _p(conv_ring), _p(q_norm), _p(k_norm), _p(freq),
+                                             0 if freq is None else 2 * freq.numel(), mag, 1 if interleaved else 0, eps, _p(ring_k), _p(ring_v), _p(sb.tok_seq), _p(sb.tok_pos), _p(sb.slots),
+                                             _p(sb.pos0), _p(sb.len_after), n, q_heads, kv_heads, dim, vdim, rows, keep_first, code(out.dtype), _stream(out)))
+
+
 def _gate_args(gate_view, n: int, heads: int, vdim: int, dtype, name: str):
     """A gate before its sigmoid: one column per head, or one per value element."""
     if gate_view is None:
@@ -492,10 +527,10 @@ def _gate_args(gate_view, n: int, heads: int, vdim: int, dtype, name: str):
 
 
 def attn_prefill_maps(out, q_view, k_view, v_view, gate_view, sink, cu, tok_seq, tok_pos, heads: int, kv_heads: int, maps: int, dim: int, vdim: int, scale: float,
-                      softcap: float, window: int, mask: int, max_rows: int = 0, mfma: bool | None = None, keep: int = 0):
+                      softcap: float, window: int, mask: int, max_rows: int = 0, mfma: bool | None = None, keep: int = 0, out_scale: float = 1.0):
     """Prompt-step attention over the step's own keys with `maps` maps per head, a soft cap and a window or chunk mask.  out [n, heads * maps * vdim] in
     float32 or the activation type, possibly a column block of a wider matrix; the gate has one column per head or one per value element; the first `keep` positions
-    stay visible beside the window.  mfma None: the matrix-core kernel for bfloat16 steps from ATTN_MFMA_MIN_ROWS rows."""
+    stay visible beside the window; the result is multiplied by out_scale.  mfma None: the matrix-core kernel for bfloat16 steps from ATTN_MFMA_MIN_ROWS rows."""
     n = q_view.shape[0]
     out_ld = _view(out, heads * maps * vdim, "out")
     _req(out.shape[0] == n and out.dtype in (torch.float32, q_view.dtype), "attn_prefill_maps: out")
@@ -510,11 +545,11 @@ def attn_prefill_maps(out, q_view, k_view, v_view, gate_view, sink, cu, tok_seq,
         _req(q_view.dtype == torch.bfloat16 and max_rows > 0, "attn_prefill_maps: the matrix-core kernel takes bfloat16 and the step's longest sequence")
         _check(_lib.mixlib().exl3_mix_attn_prefill_mfma_ex(_p(out), out_ld, out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(k_view), _view(k_view, kv_heads * maps * dim, "k"),
                                                             _p(v_view), _view(v_view, kv_heads * vdim, "v"), gate, gate_ld, gate_cols, _p(sink), _p(cu), cu.numel() - 1, max_rows,
-                                                            heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, _stream(out)))
+                                                            heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, out_scale, _stream(out)))
         return
     _check(_lib.mixlib().exl3_mix_attn_prefill_ex(_p(out), out_ld, out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(k_view), _view(k_view, kv_heads * maps * dim, "k"),
                                                    _p(v_view), _view(v_view, kv_heads * vdim, "v"), gate, gate_ld, gate_cols, _p(sink), _p(cu), _p(tok_seq), _p(tok_pos),
-                                                   n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, code(q_view.dtype), _stream(out)))
+                                                   n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, keep, out_scale, code(q_view.dtype), _stream(out)))
 
 
 def diff_mfma_ok(dtype, max_rows: int, dim: int, vdim: int, scale: float) -> bool:
@@ -535,7 +570,8 @@ def attn_prefill_diff(out, q_view, k_view, v_view, gate_view, cu, heads: int, kv
                                                           cu.numel() - 1, max_rows, heads, kv_heads, dim, vdim, scale, softcap, window, mask, lam, diff, eps, _stream(out)))
 
 
-def attn_decode_maps(out, q_view, ring_k, ring_v, gate_view, sink, slots, len_after, heads: int, maps: int, scale: float, softcap: float, mask: int):
+def attn_decode_maps(out, q_view, ring_k, ring_v, gate_view, sink, slots, len_after, heads: int, maps: int, scale: float, softcap: float, mask: int,
+                     out_scale: float = 1.0):
     """One new row per sequence against the rings (ring_k [slots, window, kv_heads * maps, dim], ring_v [slots, window, kv_heads, vdim])."""
     n = out.shape[0]
     n_slots, window, k_heads, dim = ring_k.shape
@@ -550,7 +586,7 @@ def attn_decode_maps(out, q_view, ring_k, ring_v, gate_view, sink, slots, len_af
     out_f32 = 1 if (out.dtype == torch.float32 and q_view.dtype != torch.float32) else 0
     _check(_lib.mixlib().exl3_mix_attn_decode_ex(_p(out), out_ld, out_f32, _p(q_view), _view(q_view, heads * maps * dim, "q"), _p(ring_k), _p(ring_v), gate,
                                                   gate_ld, gate_cols, _p(sink), _p(slots), _p(len_after),
-                                                  n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, code(q_view.dtype), _stream(out)))
+                                                  n, heads, kv_heads, maps, dim, vdim, scale, softcap, window, mask, out_scale, code(q_view.dtype), _stream(out)))
 
 
 def diff_combine(out, a, lam: float, diff: float, eps: float, gate_view, heads: int, vdim: int):
@@ -958,3 +994,70 @@ def retention_step(out, state, q_view, k_view, v_view, gate_view, pw, freq, inte
     a, b = _retention_args(q_view, k_view, v_view, pw, freq, heads, dim, vdim, "retention_step")
     _check(_lib.mixlib().exl3_mix_retention_step(_p(out), _view(out, heads * vdim, "out"), _p(state), *a, _p(gate_view), _view(gate_view, heads * vdim, "gate"), *b,
                                                   1 if interleaved else 0, _p(tok_pos), _p(slots), n, heads, dim, vdim, k_scale, eps, code(out.dtype), _stream(out)))
+
+
+# ---- time mixing: a decay per key channel and token, a bonus for the current token (csrc/mix_timemix.hip) --------------------------------------------
+TIMEMIX_TILE = 16             # rows of a prompt tile: segments are whole tiles
+TIMEMIX_FUSED_VDIM = 64       # head norm and gate run in the prompt kernel up to this value size
+
+
+def token_shift(out, h_view, last, mu, sb):
+    """out [mixes, n, width] = h + (h' - h) mu[m], h' the previous token's row (the step's own, or last [slots, width], or zeros); a sequence's last row goes into `last`."""
+    mixes, n, width = out.shape
+    _f32c(mu, "mu")
+    _req(out.is_contiguous() and mu.shape == (mixes, width) and h_view.shape[0] == n and last.is_contiguous() and last.dim() == 2 and last.shape[1] == width
+         and out.dtype == h_view.dtype == last.dtype, "token_shift: shapes")
+    for t, nm in ((sb.tok_seq, "tok_seq"), (sb.tok_pos, "tok_pos"), (sb.slots, "slots"), (sb.pos0, "pos0"), (sb.len_after, "len_after")):
+        _i32c(t, nm)
+    _req(sb.tok_seq.numel() == n and sb.tok_pos.numel() == n, "token_shift: rows")
+    _check(_lib.mixlib().exl3_mix_token_shift(_p(out), _p(h_view), _view(h_view, width, "h"), _p(last), _p(mu), mixes, _p(sb.tok_seq), _p(sb.tok_pos), _p(sb.slots), _p(sb.pos0),
+                                               _p(sb.len_after), n, width, code(out.dtype), _stream(out)))
+
+
+def decay_log(out, t_view, w2, w0):
+    """out [n, channels] float32 = -exp(w0 + w2 tanh(t)): the logarithms of the decays."""
+    n, channels = out.shape
+    _f32c(out, "out"); _f32c(w0, "w0")
+    _req(w2.is_contiguous() and w2.shape[0] == channels == w0.numel() and t_view.shape[0] == n and w2.dtype == t_view.dtype, "decay_log: shapes")
+    _check(_lib.mixlib().exl3_mix_decay_log(_p(out), _p(t_view), _view(t_view, w2.shape[1], "t"), _p(w2), _p(w0), n, channels, w2.shape[1], code(w2.dtype), _stream(out)))
+
+
+def timemix(o, out, gate_view, norm_w, eps: float, state, r_view, k_view, v_view, logw, u, cu, slots, pos0, segments: tuple[int, int] | None = None):
+    """Prompt steps.  state [slots, heads, dim, vdim] float32, logw [n, heads * dim] float32, u [heads * dim] float32.  Either o [n, heads, vdim] float32 receives the
+    read-outs, or (vdim <= TIMEMIX_FUSED_VDIM) out [n, heads * vdim] the heads after norm, norm_w and silu gate.  segments = (segs, seg_len): every sequence cut into parallel
+    segments; None: one chain of tiles per sequence."""
+    n = r_view.shape[0]
+    heads, dim, vdim = state.shape[1:]
+    _f32c(state, "state"); _f32c(logw, "logw"); _f32c(u, "u")
+    for t, nm in ((cu, "cu"), (slots, "slots"), (pos0, "pos0")):
+        _i32c(t, nm)
+    batch = slots.numel()
+    _req(logw.shape == (n, heads * dim) and u.numel() == heads * dim and cu.numel() == batch + 1 and pos0.numel() == batch and k_view.shape[0] == n and v_view.shape[0] == n
+         and r_view.dtype == k_view.dtype == v_view.dtype, "timemix: shapes")
+    _req((o is None) != (out is None), "timemix: either the read-outs or the gated heads")
+    oa = (None, 0, None, 0, None)
+    if out is not None:
+        _f32c(norm_w, "norm_w")
+        _req(out.shape[0] == n and gate_view.shape[0] == n and out.dtype == gate_view.dtype == r_view.dtype and norm_w.numel() == heads * vdim, "timemix: result / gate")
+        oa = (_p(out), _view(out, heads * vdim, "out"), _p(gate_view), _view(gate_view, heads * vdim, "gate"), _p(norm_w))
+    else:
+        _f32c(o, "o"); _req(o.shape == (n, heads, vdim), "timemix: o")
+    segs, seg_len = segments or (1, 0)
+    seg_state = torch.empty((batch * segs, heads, dim, vdim), dtype=torch.float32, device=state.device) if segs > 1 else None
+    seg_decay = torch.empty((batch * segs, heads, dim), dtype=torch.float32, device=state.device) if segs > 1 else None
+    _check(_lib.mixlib().exl3_mix_timemix(_p(o), *oa, eps, _p(state), _p(r_view), _view(r_view, heads * dim, "r"), _p(k_view), _view(k_view, heads * dim, "k"), _p(v_view),
+                                           _view(v_view, heads * vdim, "v"), _p(logw), _p(u), _p(cu), _p(slots), _p(pos0), batch, heads, dim, vdim, segs, seg_len, _p(seg_state),
+                                           _p(seg_decay), code(r_view.dtype), _stream(state)))
+
+
+def timemix_step(out, state, r_view, k_view, v_view, gate_view, t_view, w2, w0, u, norm_w, tok_pos, slots, eps: float):
+    """One row per sequence: decays from the low-rank input t, read-out, state update, head norm, norm_w and silu gate in one launch; out [n, heads * vdim]."""
+    n = out.shape[0]
+    heads, dim, vdim = state.shape[1:]
+    _f32c(state, "state"); _f32c(w0, "w0"); _f32c(u, "u"); _f32c(norm_w, "norm_w"); _i32c(tok_pos, "tok_pos"); _i32c(slots, "slots")
+    _req(slots.numel() == n and tok_pos.numel() == n and all(t.shape[0] == n and t.dtype == out.dtype for t in (r_view, k_view, v_view, gate_view, t_view)) and w2.is_contiguous()
+         and w2.dtype == out.dtype and w2.shape[0] == heads * dim == w0.numel() == u.numel() and norm_w.numel() == heads * vdim, "timemix_step: shapes")
+    _check(_lib.mixlib().exl3_mix_timemix_step(_p(out), _view(out, heads * vdim, "out"), _p(state), _p(r_view), _view(r_view, heads * dim, "r"), _p(k_view), _view(k_view, heads * dim, "k"),
+                                                _p(v_view), _view(v_view, heads * vdim, "v"), _p(gate_view), _view(gate_view, heads * vdim, "gate"), _p(t_view),
+                                                _view(t_view, w2.shape[1], "t"), _p(w2), _p(w0), _p(u), _p(norm_w), _p(tok_pos), _p(slots), n, heads, dim, vdim, w2.shape[1], eps,
+                                                code(out.dtype), _stream(out)))

@@ -40,8 +40,13 @@ float32 accumulation; true float32 when the model runs in float32).
     PagedLatentAttention    latent attention without a window: the cached rows live in the cache's pages; queries through a normed latent of their own; either
                             pairing of the rotation; a layer may read another layer's cached rows instead of having any
     KeptWindowAttention     grouped-query attention over a sliding window beside which the first tokens of a sequence stay visible; rotated queries and keys, values
-                            of their own or the keys before their rotation; sink, output gate per value element
+                            of their own or the keys before their rotation; sink, output gate per value element; short convolutions on q / k / v, normed queries
+                            and keys, soft-capped scores
     Retention               linear attention with a fixed decay per head, rotated queries and keys, float32 state, per-head unit RMS, silu gate
+    TimeMix                 RWKV-style time mixing: token shift, a decay per key channel and token from a low-rank product, a bonus for the current token, float32 state,
+                            per-head unit RMS, silu gate
+    SummedMixers            two mixers side by side, scaled and added inside ONE output product
+    PostNormBlock           x += norm1(mixer(x)); x += norm2(ff(x)): the norms sit on the sublayers' outputs, which read the stream itself
     DualNormBlock           x += mixer(norm1(x)) + ff(norm2(x)): both norms from one pass over the stream, both output projections as ONE product over
                             [mixer's heads | hidden activation]
 
@@ -201,12 +206,19 @@ class PolyNormMLP:
 def rotary_frequencies(dims: int, base: float, scaling: dict | None = None) -> tuple[torch.Tensor, float]:
     """Per-pair frequencies base^(-2i/dims), i < dims/2, and the magnitude that multiplies cos and sin.  `scaling` (YaRN: factor, original, fast, slow)
     blends every frequency with its `factor`-times slower version along a linear ramp between the pair indices at which the original context
-    holds `fast` and `slow` turns, and sets the magnitude to 0.1 ln(factor) + 1.  Computed in float64, returned as float32."""
+    holds `fast` and `slow` turns, and sets the magnitude to 0.1 ln(factor) + 1.  `scaling` with bounds in turns (Llama 3.1: factor, original, low, high): a pair that turns
+    more than `high` times over the original context keeps its frequency, one that turns less than `low` times gets 1 / factor of it, those between are blended by their
+    turns; the magnitude stays 1.  Computed in float64, returned as float32."""
     import math
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = float(base) ** (-2.0 * i / dims)
     mag = 1.0
-    if scaling is not None:
+    if scaling is not None and "low" in scaling:
+        factor, original, low, high = (float(scaling[nm]) for nm in ("factor", "original", "low", "high"))
+        length = 2.0 * math.pi / f                               # positions per turn
+        s = (original / length - low) / (high - low) if high != low else torch.zeros_like(f)
+        f = torch.where(length < original / high, f, torch.where(length > original / low, f / factor, (1.0 - s) * f / factor + s * f))
+    elif scaling is not None:
         factor, original = float(scaling["factor"]), float(scaling["original"])
         at = lambda turns: dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(float(base)))
         lo = max(math.floor(at(float(scaling["fast"]))), 0)
@@ -328,9 +340,12 @@ class PagedLatentAttention(LatentAttention):
     of the same step, handed over in the step's `shared` dict, in decode steps that layer's pages."""
 
     def __init__(self, width: int, heads: int, dim: int, rot_dim: int, vdim: int, rank: int, q_rank: int, scale: float, eps: float, rot_dims: int, rot_base: float,
-                 rot_scaling: dict | None = None, interleaved: bool = False, sink: bool = False, gate: bool = False, layer: int = 0, kv_from: int | None = None):
+                 rot_scaling: dict | None = None, interleaved: bool = False, sink: bool = False, gate: bool = False, layer: int = 0, kv_from: int | None = None,
+                 gate_per_head: bool = False):
+        """gate: the heads times sigmoid(W_g h), one number per value element, or (gate_per_head) one per head."""
         super().__init__(width, heads, dim, rot_dim, vdim, rank, scale, 1, eps, rot_dims, rot_base, rot_scaling, sink, gate)
         self.q_rank, self.interleaved, self.layer, self.kv_from = int(q_rank), bool(interleaved), layer, kv_from
+        self.gate_cols = heads if gate_per_head else heads * vdim
         self.out_width = heads * vdim
 
     EVERY = 1 << 30                          # a window that no sequence reaches the end of
@@ -342,6 +357,7 @@ class PagedLatentAttention(LatentAttention):
         if self.has_gate:
             parts.append(("g", _w(stc, prefix + "g", dtype, device), None))
         self.inp = FusedInput(parts + list(extra_parts))
+        assert not self.has_gate or self.inp.offsets["g"][1] == self.gate_cols
         self.q_norm, self.w_uq = _f32(stc, prefix + "dq.norm", device), _w(stc, prefix + "uq", dtype, device)
         assert self.inp.offsets["dq"][1] == self.q_rank == self.q_norm.numel() and self.w_uq.shape == (self.heads * self.qk, self.q_rank)
         if self.kv_from is None:
@@ -391,13 +407,16 @@ class PagedLatentAttention(LatentAttention):
 
 
 class KeptWindowAttention:
-    """H query heads over G key/value heads, no biases.  A row sees the last `size` positions up to itself and the sequence's first `keep_first` positions, which keep
+    """H query heads over G key/value heads.  A row sees the last `size` positions up to itself and the sequence's first `keep_first` positions, which keep
     their true positions.  Rotary positions on the first rot_dims entries of queries and keys; tied: the values are the keys before their rotation (no W_v).
     Optional sink (one more term of the denominator per head) and output gate per value element.  A slot holds keep_first + size rows of keys and values: the
-    first positions' for good, and a ring of the last `size` of the others."""
+    first positions' for good, and a ring of the last `size` of the others.  Optional: biases of the q / k / v projections; a short causal convolution over time on every
+    channel of q, k and v (taps > 0; the slot also holds the last taps - 1 projected rows); an RMS norm of every query / key head with a plain weight over dim; scores
+    soft-capped to softcap tanh(score / softcap); a factor on the result (out_scale)."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, size: int, keep_first: int, rot_dims: int, rot_base: float,
-                 interleaved: bool = True, tied: bool = False, sink: bool = True, gate: bool = True):
+                 interleaved: bool = True, tied: bool = False, sink: bool = True, gate: bool = True, bias: bool = False, taps: int = 0, qk_norm: bool = False, softcap: float = 0.0,
+                 rot_scaling: dict | None = None, eps: float = 0.0, out_scale: float = 1.0):
         if heads % kv_heads:
             raise RuntimeError(f"attention: {heads} query heads over {kv_heads} key/value heads")
         if tied and dim != vdim:
@@ -407,35 +426,59 @@ class KeptWindowAttention:
         self.width, self.heads, self.kv_heads, self.dim, self.vdim, self.scale = width, heads, kv_heads, dim, vdim, float(scale)
         self.size, self.keep_first, self.rot_dims, self.rot_base, self.interleaved = int(size), int(keep_first), int(rot_dims), float(rot_base), bool(interleaved)
         self.tied, self.has_sink, self.has_gate = tied, sink, gate
+        if taps and (tied or not 1 <= taps <= 16):
+            raise RuntimeError(f"attention: a convolution of {taps} taps (1 to 16, values of their own)")
+        self.has_bias, self.taps, self.has_qk_norm, self.softcap, self.rot_scaling, self.eps = bias, int(taps), qk_norm, float(softcap or 0.0), rot_scaling, float(eps)
+        self.out_scale = float(out_scale)
         self.out_width = heads * vdim
+        self.channels = heads * dim + kv_heads * (dim + vdim)
 
     def load(self, stc, prefix: str, dtype, device, extra_parts=()):
         names = ["q", "k"] + ([] if self.tied else ["v"]) + (["g"] if self.has_gate else [])
-        self.inp = FusedInput([(nm, _w(stc, prefix + nm, dtype, device), None) for nm in names] + list(extra_parts))
+        bias = lambda nm: _w(stc, prefix + nm + ".b", dtype, device) if self.has_bias and nm != "g" else None
+        self.inp = FusedInput([(nm, _w(stc, prefix + nm, dtype, device), bias(nm)) for nm in names] + list(extra_parts))
         self.sink = _f32(stc, prefix + "sink", device) if self.has_sink else None
         self.w_o = _w(stc, prefix + "o", dtype, device)
         assert self.inp.offsets["q"][1] == self.heads * self.dim and self.inp.offsets["k"][1] == self.kv_heads * self.dim
+        assert (self.tied or self.inp.offsets["v"][1] == self.kv_heads * self.vdim) and (not self.has_gate or self.inp.offsets["g"][1] == self.out_width)
         assert self.w_o.shape == (self.width, self.out_width)
-        self.freq = rotary_frequencies(self.rot_dims, self.rot_base)[0].to(device).contiguous() if self.rot_dims else None
+        self.q_norm, self.k_norm = (_f32(stc, prefix + nm, device) if self.has_qk_norm else None for nm in ("q.norm", "k.norm"))
+        self.conv = None
+        if self.taps:                                            # stored [channels, taps] per projection; the kernel reads one tap of neighbouring channels at once
+            self.conv = torch.cat([_f32(stc, prefix + nm + ".conv", device) for nm in ("q", "k", "v")], dim=0).t().contiguous()
+            assert self.conv.shape == (self.taps, self.channels)
+        self.freq, self.rot_mag = None, 1.0
+        if self.rot_dims:
+            f, self.rot_mag = rotary_frequencies(self.rot_dims, self.rot_base, self.rot_scaling)
+            self.freq = f.to(device).contiguous()
         self.dtype = dtype
 
     def state_specs(self) -> list:
         rows = self.keep_first + self.size
-        return [StateSpec("ring_k", (rows, self.kv_heads, self.dim), self.dtype), StateSpec("ring_v", (rows, self.kv_heads, self.vdim), self.dtype)]
+        specs = [StateSpec("ring_k", (rows, self.kv_heads, self.dim), self.dtype), StateSpec("ring_v", (rows, self.kv_heads, self.vdim), self.dtype)]
+        return specs + ([StateSpec("conv", (max(self.taps - 1, 1), self.channels), self.dtype)] if self.taps else [])
 
     def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
         H, G, d, dv = self.heads, self.kv_heads, self.dim, self.vdim
         p = self.inp(h)
         q, k = p["q"], p["k"]
         v = k if self.tied else p["v"]
-        k_rot = torch.empty((sb.n, G * d), dtype=self.dtype, device=h.device) if self.tied else None
-        mix_ops.qk_prep(q, k, v, None, None, self.freq, 1.0, self.interleaved, 0.0, state["ring_k"], state["ring_v"], sb.tok_seq, sb.tok_pos, sb.slots, sb.len_after, d,
-                        k_out=k_rot, keep_first=self.keep_first)
-        if sb.decode:
-            mix_ops.attn_decode_maps(out, q, state["ring_k"], state["ring_v"], p.get("g"), self.sink, sb.slots, sb.len_after, H, 1, self.scale, 0.0, mix_ops.MASK_WINDOW)
+        if self.taps:
+            z = torch.empty((sb.n, self.channels), dtype=self.dtype, device=h.device)
+            mix_ops.conv_prep(z, self.inp.block(p, "q", "v"), self.conv, state["conv"], self.q_norm, self.k_norm, self.freq, self.rot_mag, self.interleaved, self.eps, state["ring_k"],
+                              state["ring_v"], sb, H, keep_first=self.keep_first)
+            q, k, v = z[:, : H * d], z[:, H * d: (H + G) * d], z[:, (H + G) * d:]
         else:
-            mix_ops.attn_prefill_maps(out, q, k_rot if self.tied else k, v, p.get("g"), self.sink, sb.cu, sb.tok_seq, sb.tok_pos, H, G, 1, d, dv, self.scale, 0.0, self.size,
-                                      mix_ops.MASK_WINDOW, max_rows=sb.max_rows, keep=self.keep_first)
+            k_rot = torch.empty((sb.n, G * d), dtype=self.dtype, device=h.device) if self.tied else None
+            mix_ops.qk_prep(q, k, v, self.q_norm, self.k_norm, self.freq, self.rot_mag, self.interleaved, self.eps, state["ring_k"], state["ring_v"], sb.tok_seq, sb.tok_pos, sb.slots,
+                            sb.len_after, d, k_out=k_rot, keep_first=self.keep_first)
+            k = k_rot if self.tied else k
+        if sb.decode:
+            mix_ops.attn_decode_maps(out, q, state["ring_k"], state["ring_v"], p.get("g"), self.sink, sb.slots, sb.len_after, H, 1, self.scale, self.softcap, mix_ops.MASK_WINDOW,
+                                     out_scale=self.out_scale)
+        else:
+            mix_ops.attn_prefill_maps(out, q, k, v, p.get("g"), self.sink, sb.cu, sb.tok_seq, sb.tok_pos, H, G, 1, d, dv, self.scale, self.softcap, self.size,
+                                      mix_ops.MASK_WINDOW, max_rows=sb.max_rows, keep=self.keep_first, out_scale=self.out_scale)
 
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
@@ -493,6 +536,106 @@ class Retention:
         o = torch.empty((sb.n, self.heads, self.vdim), dtype=torch.float32, device=h.device)
         mix_ops.retention(o, state["S"], p["q"], p["k"], p["v"], self.pw, self.freq, self.interleaved, sb.cu, sb.slots, sb.pos0, self.k_scale, segments=self.segments(sb))
         mix_ops.head_norm_gate(out, o, None, p["g"], mix_ops.GATE_SILU, self.eps)
+
+    def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
+        out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
+        self.attend(h, sb, state, out)
+        return F.linear(out, self.w_o)
+
+
+class TimeMix:
+    """RWKV-style time mixing.  With h' the previous token's h (zeros ahead of the first), each of r, k, v, g, w reads its own mix h + (h' - h) mu; r, k, v per head, gate =
+    silu(W_g mix_g); decay w = exp(-exp(w0 + W_w2 tanh(W_w1 mix_w))) per head and key channel.  o_t = (S + diag(u) k v^T)^T r, then S <- diag(w) S + k v^T; each head's o over
+    its root mean square, times a weight over all heads' values, times the gate.  Per slot: S [heads, dim, dim] float32 and the last token's h.  out_scale: a factor
+    on the result (folded into the float32 weight)."""
+    # prompt steps whose longest sequence has at least this many rows are cut into parallel segments, enough of them for about this many workgroups
+    SEGMENT_MIN_ROWS = 256
+    SEGMENT_TARGET_WORKGROUPS = 1024
+    SEGMENT_ROWS = 64                        # a segment's shortest length
+
+    def __init__(self, width: int, heads: int, dim: int, eps: float, out_scale: float = 1.0):
+        if dim > 256:
+            raise RuntimeError("time mixing: a head has at most 256 key channels")
+        self.width, self.heads, self.dim, self.eps, self.out_scale = width, heads, dim, float(eps), float(out_scale)
+        self.out_width = heads * dim
+        self.dtype = torch.bfloat16                                  # until load() says otherwise
+
+    def load(self, stc, prefix: str, dtype, device, extra_parts=()):
+        self.inp = FusedInput(list(extra_parts)) if extra_parts else None
+        n = self.heads * self.dim
+        # r, k, v, g as one batched product over their mixes: [4, width, heads * dim]
+        self.w_rkvg = torch.stack([_w(stc, prefix + nm, dtype, device).t() for nm in ("r", "k", "v", "g")]).contiguous()
+        self.mu = torch.stack([_f32(stc, prefix + "mu." + nm, device) for nm in ("r", "k", "v", "g", "w")]).contiguous()
+        self.w1, self.w2 = _w(stc, prefix + "w1", dtype, device), _w(stc, prefix + "w2", dtype, device)
+        self.w0, self.u = _f32(stc, prefix + "w0", device), _f32(stc, prefix + "u", device).reshape(-1).contiguous()
+        self.norm_w = (_f32(stc, prefix + "norm", device) * self.out_scale).contiguous()
+        self.w_o = _w(stc, prefix + "o", dtype, device)
+        assert self.w_rkvg.shape == (4, self.width, n) and self.mu.shape == (5, self.width) and self.w1.shape == (self.w2.shape[1], self.width) and self.w2.shape[0] == n
+        assert self.w0.numel() == self.u.numel() == self.norm_w.numel() == n and self.w_o.shape == (self.width, n)
+        self.dtype = dtype
+
+    def state_specs(self) -> list:
+        return [StateSpec("S", (self.heads, self.dim, self.dim), torch.float32), StateSpec("last", (self.width,), self.dtype)]
+
+    def segments(self, sb: StepBatch) -> tuple[int, int] | None:
+        if sb.max_rows < self.SEGMENT_MIN_ROWS:
+            return None
+        chains = sb.batch * self.heads * ((self.dim + 63) // 64)
+        segs = min(-(-self.SEGMENT_TARGET_WORKGROUPS // chains), sb.max_rows // self.SEGMENT_ROWS)
+        if segs < 2:
+            return None
+        tile = mix_ops.TIMEMIX_TILE
+        seg_len = -(-(-(-sb.max_rows // segs)) // tile) * tile
+        return -(-sb.max_rows // seg_len), seg_len
+
+    def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
+        mix = torch.empty((5, sb.n, self.width), dtype=self.dtype, device=h.device)
+        mix_ops.token_shift(mix, h, state["last"], self.mu, sb)
+        r, k, v, g = torch.bmm(mix[:4], self.w_rkvg).unbind(0)
+        t = F.linear(mix[4], self.w1)
+        if sb.decode:
+            mix_ops.timemix_step(out, state["S"], r, k, v, g, t, self.w2, self.w0, self.u, self.norm_w, sb.tok_pos, sb.slots, self.eps)
+            return
+        logw = torch.empty((sb.n, self.out_width), dtype=torch.float32, device=h.device)
+        mix_ops.decay_log(logw, t, self.w2, self.w0)
+        fused = self.dim <= mix_ops.TIMEMIX_FUSED_VDIM
+        o = None if fused else torch.empty((sb.n, self.heads, self.dim), dtype=torch.float32, device=h.device)
+        mix_ops.timemix(o, out if fused else None, g, self.norm_w, self.eps, state["S"], r, k, v, logw, self.u, sb.cu, sb.slots, sb.pos0, segments=self.segments(sb))
+        if not fused:
+            mix_ops.head_norm_gate(out, o, self.norm_w, g, mix_ops.GATE_SILU, self.eps)
+
+    def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
+        out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
+        self.attend(h, sb, state, out)
+        return F.linear(out, self.w_o)
+
+
+class SummedMixers:
+    """Two mixers side by side that read the same input, result = left + right (factors of the two are the mixers' own out_scale).  Both write their heads into column blocks
+    of one matrix and their output projections are one product over it: the sum is a float32 accumulation."""
+
+    def __init__(self, width: int, left, right):
+        self.width, self.left, self.right = width, left, right
+        self.out_width = left.out_width + right.out_width
+
+    def load(self, stc, prefix: str, dtype, device, extra_parts=()):
+        self.left.load(stc, prefix + "left.", dtype, device, extra_parts)
+        self.right.load(stc, prefix + "right.", dtype, device)
+        at = self.left.out_width
+        self.w_o = torch.cat([self.left.w_o, self.right.w_o], dim=1).contiguous()
+        self.left.w_o, self.right.w_o = self.w_o[:, :at], self.w_o[:, at:]              # views: the weights are held once
+        self.dtype = dtype
+
+    def state_specs(self) -> list:
+        specs = self.left.state_specs() + self.right.state_specs()
+        if len({s.name for s in specs}) != len(specs):
+            raise RuntimeError("parallel mixers: both sides would keep a state of the same name")
+        return specs
+
+    def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
+        at = self.left.out_width
+        self.left.attend(h, sb, state, out[:, :at])
+        self.right.attend(h, sb, state, out[:, at:])
 
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
@@ -1121,3 +1264,37 @@ class DualNormBlock:
         if self.mlp is not None:
             self.mlp.hidden(h2, out=cat[:, self.split:])
         return F.linear(cat, self.w_out)
+
+
+class PostNormBlock:
+    """x <- x + norm1(mixer(x)), then x <- x + norm2(ff(x)) (if a feed-forward): RMS norms on the sublayers' outputs, whose stored weights are deviations from one; the
+    sublayers read the float32 stream itself, in the activation type.  Every update of the stream is one kernel: the norm of the sublayer's output, the addition and
+    the copy of the stream that the next sublayer reads."""
+
+    def __init__(self, width: int, eps: float, mixer, mlp):
+        self.width, self.eps, self.mixer, self.mlp = width, float(eps), mixer, mlp
+
+    def load(self, stc, prefix: str, dtype, device):
+        self.norm1 = (1.0 + _f32(stc, prefix + "norm1", device)).contiguous()
+        self.norm2 = None
+        self.mixer.load(stc, prefix + "mix.", dtype, device)
+        assert self.norm1.numel() == self.width
+        if self.mlp is not None:
+            self.norm2 = (1.0 + _f32(stc, prefix + "norm2", device)).contiguous()
+            self.mlp.load(stc, prefix + "mlp.", dtype, device)
+            assert self.norm2.numel() == self.width
+        self.dtype = dtype
+
+    def state_specs(self) -> list:
+        return self.mixer.state_specs()
+
+    def forward(self, x: torch.Tensor, h: torch.Tensor, sb: StepBatch, state: dict, last: bool = False) -> torch.Tensor | None:
+        """x: float32 residual (updated in place); h: x in the activation type.  Returns the stream after the block in the activation type (None if `last`)."""
+        def update(y, w, out):
+            update_residual(x, y, None if out is None else NextInput(None, out), rms_w=w, eps=self.eps)
+            return out
+        new = lambda skip: None if skip else torch.empty_like(h)
+        h = update(self.mixer.forward(h, sb, state), self.norm1, new(last and self.mlp is None))
+        if self.mlp is not None:
+            h = update(self.mlp.forward(h, sb)[0], self.norm2, new(last))
+        return h

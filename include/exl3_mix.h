@@ -48,7 +48,7 @@ extern "C" {
 #define EXL3_MIX_MASK_WINDOW 0
 #define EXL3_MIX_MASK_CHUNK  1
 
-#define EXL3_MIX_ABI_VERSION 5
+#define EXL3_MIX_ABI_VERSION 6
 
 const char* exl3_mix_last_error(void);
 int  exl3_mix_abi_version(void);
@@ -150,6 +150,9 @@ int exl3_mix_moe_expert_major_act(void* per, void* hid, const void* h, const voi
 /* x[n] = table[tokens[n]] (float32 residual); if xc: the same row in the activation type at xc + n * xc_ld. */
 int exl3_mix_embed_copy(float* x, void* xc, int64_t xc_ld, const void* table, const int32_t* tokens, int n, int width, int vocab, int dtype, void* stream);
 
+/* x[n] = t / sqrt(mean(t^2) + eps) * w with t = table[tokens[n]] (float32 residual); if xc: the same row in the activation type. */
+int exl3_mix_embed_norm(float* x, void* xc, int64_t xc_ld, const void* table, const int32_t* tokens, const float* w, float eps, int n, int width, int vocab, int dtype, void* stream);
+
 /* Residual update fused with what the next consumer reads.  mode 0: x stays (y unused); 1: x += y'; 2: x = y', where y' = y, or, with rms_w,
  * y / sqrt(mean(y^2) + eps) * rms_w.  out 0: nothing; 1: h = x in the activation type; 2: h = tanh(alpha x) * w + b (Dynamic Tanh: no mean, no
  * variance).  y and h may be column blocks (row strides y_ld, h_ld). */
@@ -167,9 +170,9 @@ int exl3_mix_glu_act(void* out, const void* g, int64_t g_ld, const void* u, int6
 int exl3_mix_token_gate(void* out, const void* gate, int64_t gate_ld, const void* table, int64_t table_ld, int col0, const int32_t* tokens,
                         int n, int dim, int vocab, int dtype, void* stream);
 
-/* out[n][h * vdim + v] = a[n * a_row + h * a_head + v] * (gate ? sigmoid(gate[n][h * vdim + v]) : 1): an element-wise output gate over heads that may lie
- * head-major (the result of a per-head batched product). */
-int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int n, int heads, int vdim, int dtype, void* stream);
+/* out[n][h * vdim + v] = a[n * a_row + h * a_head + v] * (gate ? sigmoid(gate[n][h * vdim + v]) : 1): an output gate over heads that may lie head-major (the
+ * result of a per-head batched product); the gate has gate_cols = vdim columns per head, or gate_cols = 1. */
+int exl3_mix_heads_gate(void* out, int64_t out_ld, const void* a, int64_t a_row, int64_t a_head, const void* gate, int64_t gate_ld, int gate_cols, int n, int heads, int vdim, int dtype, void* stream);
 
 /* Router with independent scores s = sigmoid(z): the `top` experts with the largest s + correction (correction may be NULL; ties go to the lower index);
  * weights = s / (sum of the chosen s + 1e-20) * scale, or s * scale with normalise = 0. */
@@ -222,17 +225,18 @@ int exl3_mix_rotate_heads(void* q, int64_t q_ld, const int32_t* tok_pos, const f
  * of the head's key/value head; out [n][heads][maps][vdim]; a gate needs maps == 1), scores soft-capped to softcap tanh(score / softcap) (softcap 0: none),
  * mask EXL3_MIX_MASK_* over `window` positions, values as a column block (v_ld), and the result in float32 (out_f32) or the activation type.
  * Decode with the chunk mask reads the ring entries 0 .. (len_after - 1) % window.  out is a column block (row stride out_ld); the gate has gate_cols = 1 column per head
- * or gate_cols = vdim columns per head (one per value element); keep (prompt steps, window mask): the first `keep` positions stay visible beside the window. */
+ * or gate_cols = vdim columns per head (one per value element); keep (prompt steps, window mask): the first `keep` positions stay visible beside the window;
+ * the result is multiplied by out_scale. */
 int exl3_mix_attn_prefill_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
                              const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu, const int32_t* tok_seq, const int32_t* tok_pos,
-                             int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, int dtype, void* stream);
+                             int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep, float out_scale, int dtype, void* stream);
 int exl3_mix_attn_prefill_mfma_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
                                   const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* cu,
                                   int batch, int max_rows, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int keep,
-                                  void* stream);
+                                  float out_scale, void* stream);
 int exl3_mix_attn_decode_ex(void* out, int64_t out_ld, int out_f32, const void* q, int64_t q_ld, const void* ring_k, const void* ring_v,
                             const void* gate, int64_t gate_ld, int gate_cols, const float* sink, const int32_t* slots, const int32_t* len_after,
-                            int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, int dtype, void* stream);
+                            int n, int heads, int kv_heads, int maps, int dim, int vdim, float scale, float softcap, int window, int mask, float out_scale, int dtype, void* stream);
 
 /* Differential attention of a prompt step on the matrix cores, bfloat16 only: both maps of a head in one workgroup (the value tile is staged once for both)
  * and the combination in the epilogue: out[n][h] = rms_unit(a1 - lambda a2) (1 - diff) sigmoid(gate[n][h]) (exl3_mix_diff_combine), with a1 / a2 the
@@ -252,6 +256,14 @@ int exl3_mix_qk_prep(void* q, int64_t q_ld, const void* k, int64_t k_ld, void* k
                      const float* freq, int rot_dims, float mag, int interleaved, float eps, void* ring_k, void* ring_v,
                      const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, const int32_t* len_after,
                      int n, int q_heads, int k_heads, int v_heads, int dim, int vdim, int window, int keep_first, int dtype, void* stream);
+
+/* The same for queries, keys and values whose projections pass a short causal convolution over time (mix_convprep.hip).  x [n][q_heads dim | kv_heads dim |
+ * kv_heads vdim] (row stride x_ld); conv_w [taps][C] over those C columns, the last tap is the row's own; predecessors come from the step's own rows or from
+ * conv_ring [slots][taps - 1][C], which keeps the last taps - 1 projected rows of a sequence; zeros before its start.  out [n][C]: normed and rotated
+ * queries and keys, convolved values.  ring_k [slots][rows][kv_heads][dim], ring_v [slots][rows][kv_heads][vdim] as above (keep_first).  1..16 taps. */
+int exl3_mix_conv_prep(void* out, const void* x, int64_t x_ld, const float* conv_w, int taps, void* conv_ring, const float* q_norm, const float* k_norm, const float* freq,
+                       int rot_dims, float mag, int interleaved, float eps, void* ring_k, void* ring_v, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots,
+                       const int32_t* pos0, const int32_t* len_after, int n, int q_heads, int kv_heads, int dim, int vdim, int rows, int keep_first, int dtype, void* stream);
 
 /* Differential attention: a [n][heads][2][vdim] float32 (the two maps of every head);  o = a1 - lambda a2;
  * out[n][h][c] = o_c / sqrt(mean_c(o^2) + eps) * (1 - diff) * sigmoid(gate[n][h])  (gate NULL: no gate). */
@@ -372,6 +384,26 @@ int exl3_mix_retention(float* o, float* state, const void* q, int64_t q_ld, cons
 int exl3_mix_retention_step(void* out, int64_t out_ld, float* state, const void* q, int64_t q_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld,
                             const void* gate, int64_t gate_ld, const float* pw, int pw_ld, const float* freq, int rot_dims, int interleaved, const int32_t* tok_pos,
                             const int32_t* slots, int n, int heads, int dim, int vdim, float k_scale, float eps, int dtype, void* stream);
+
+/* ---- time mixing with a decay per key channel and token and a bonus for the current token (mix_timemix.hip) ---- */
+
+/* out[m][n] = h[n] + (h'[n] - h[n]) mu[m], m < mixes; h'[n]: the row before n in its sequence -- the step's own, or `last` [slots][width], or zeros ahead of the
+ * first token.  A sequence's last row goes into `last`.  out [mixes][n][width], mu [mixes][width]. */
+int exl3_mix_token_shift(void* out, const void* h, int64_t h_ld, void* last, const float* mu, int mixes, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots,
+                         const int32_t* pos0, const int32_t* len_after, int n, int width, int dtype, void* stream);
+/* Logarithms of the decays: out[n][c] = -exp(w0[c] + sum_r tanh(t[n][r]) w2[c][r]), c < channels (float32 throughout). */
+int exl3_mix_decay_log(float* out, const void* t, int64_t t_ld, const void* w2, const float* w0, int n, int channels, int rank, int dtype, void* stream);
+/* Per head o_t = (S + diag(u) k_t v_t^T)^T r_t, then S <- diag(w_t) S + k_t v_t^T with w = exp(logw) [n][heads * dim], u [heads * dim].  o [n][heads][vdim] float32, or
+ * with `out` (vdim <= 64) the heads after norm and gate, o / sqrt(mean(o^2) + eps) * norm_w[heads * vdim] * silu(gate).  state [slots][heads][dim][vdim] float32;
+ * dim <= 256, vdim <= 1024.  segs > 1: every sequence in `segs` segments of seg_len rows that run in parallel; seg_state holds batch * segs * heads * dim * vdim floats,
+ * seg_decay batch * segs * heads * dim. */
+int exl3_mix_timemix(float* o, void* out, int64_t out_ld, const void* gate, int64_t gate_ld, const float* norm_w, float eps, float* state, const void* r, int64_t r_ld,
+                     const void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* logw, const float* u, const int32_t* cu, const int32_t* slots,
+                     const int32_t* pos0, int batch, int heads, int dim, int vdim, int segs, int seg_len, float* seg_state, float* seg_decay, int dtype, void* stream);
+/* One row per sequence: decays (as exl3_mix_decay_log), read-out, state update, head norm and gate. */
+int exl3_mix_timemix_step(void* out, int64_t out_ld, float* state, const void* r, int64_t r_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, const void* gate,
+                          int64_t gate_ld, const void* t, int64_t t_ld, const void* w2, const float* w0, const float* u, const float* norm_w, const int32_t* tok_pos,
+                          const int32_t* slots, int n, int heads, int dim, int vdim, int rank, float eps, int dtype, void* stream);
 
 /* out[n] = scale (a[n] / rms(a[n]) * wa + b[n] / rms(b[n]) * wb). */
 int exl3_mix_rms_pair(void* out, const void* a, int64_t a_ld, const float* wa, const void* b, int64_t b_ld, const float* wb, float scale, float eps, int n, int width,
