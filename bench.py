@@ -63,7 +63,9 @@ def parse():
                     help="instead of the default workload: layer times of the parallel-block family (Dikopel) beside Vofanex layers of equal size, and its kernels' rooflines")
     ap.add_argument("--dual-family", action="store_true",
                     help="instead of the default workload: layer times of the dual-norm family (Luzinex) beside Zagilorn and Vofanex layers of equal size, and its kernels' rooflines")
-    ap.add_argument("--mixer-sizes", default="", help="with --mixer-family / --latent-family / --diff-family / --parallel-family / --dual-family: comma-separated sizes (1b, 8b; default both)")
+    ap.add_argument("--postnorm-family", action="store_true",
+                    help="instead of the default workload: layer times of the post-norm family (Menerax) beside Luzinex layers of equal size, and its kernels' rooflines")
+    ap.add_argument("--mixer-sizes", default="", help="with --mixer-family / --latent-family / --diff-family / --parallel-family / --dual-family / --postnorm-family: comma-separated sizes (1b, 8b; default both)")
     ap.add_argument("--variant", type=int, default=1)
     ap.add_argument("--attention", action="store_true", help="include decode attention over the quantized KV cache (context = 1000 tokens) in the timed step")
     ap.add_argument("--unfused", action="store_true", help="one launch per reference op instead of the fused pipeline")
@@ -274,6 +276,9 @@ def main():
     if args.dual_family:
         from exllamav3_amd import dual_bench
         sys.exit(dual_bench.run(args))
+    if args.postnorm_family:
+        from exllamav3_amd import postnorm_bench
+        sys.exit(postnorm_bench.run(args))
     import torch
     from exllamav3_amd import ext
     from exllamav3_amd.llama_path import SHAPES, SyntheticEXL3Llama

@@ -360,8 +360,9 @@ def _declare_mix(l):
     sig("exl3_mix_head_norm_gate", vp, i64, vp, vp, i32, vp, i64, i32, f32, i32, i32, i32, i32, vp)
     sig("exl3_mix_embed_norm", vp, vp, i64, vp, vp, vp, f32, i32, i32, i32, i32, vp)
     sig("exl3_mix_conv_prep", vp, vp, i64, vp, i32, vp, vp, vp, vp, i32, f32, i32, f32, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, vp)
+    sig("exl3_mix_skinny", vp, i64, i64, vp, i64, vp, i64, i64, vp, i64, vp, i32, i32, i32, i32, i32, vp)
     sig("exl3_mix_token_shift", vp, vp, i64, vp, vp, i32, vp, vp, vp, vp, vp, i32, i32, i32, vp)
-    sig("exl3_mix_decay_log", vp, vp, i64, vp, vp, i32, i32, i32, i32, vp)
+    sig("exl3_mix_decay_log2", vp, vp, i64, vp, vp, i32, i32, i32, i32, vp)
     sig("exl3_mix_timemix", vp, vp, i64, vp, i64, vp, f32, vp, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp, vp, i32, vp)
     sig("exl3_mix_timemix_step", vp, i64, vp, vp, i64, vp, i64, vp, i64, vp, i64, vp, i64, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, i32, vp)
     sig("exl3_mix_rms_pair", vp, vp, i64, vp, vp, i64, vp, f32, f32, i32, i32, i32, vp)

@@ -12,6 +12,34 @@
 #define CP_CHANNELS 1024
 #define CP_MAX_TAPS 16
 
+// V neighbouring floats in pieces of four (16-byte aligned where V is a multiple of four)
+template <int V> __device__ __forceinline__ void load_f(const float* p, float (&o)[V])
+{
+    if constexpr (V % 4 == 0)
+    {
+        #pragma unroll
+        for (int a = 0; a < V; a += 4) { const float4 t = *(const float4*) (p + a); o[a] = t.x; o[a + 1] = t.y; o[a + 2] = t.z; o[a + 3] = t.w; }
+    }
+    else
+    {
+        #pragma unroll
+        for (int e = 0; e < V; ++e) o[e] = p[e];
+    }
+}
+template <int V> __device__ __forceinline__ void store_f(float* p, const float (&o)[V])
+{
+    if constexpr (V % 4 == 0)
+    {
+        #pragma unroll
+        for (int a = 0; a < V; a += 4) *(float4*) (p + a) = make_float4(o[a], o[a + 1], o[a + 2], o[a + 3]);
+    }
+    else
+    {
+        #pragma unroll
+        for (int e = 0; e < V; ++e) p[e] = o[e];
+    }
+}
+
 // V: channels per thread and access; R: rows per workgroup; TAPS: number of taps, 0: read from `taps` (weights are then read per row)
 template <typename T, int V, int R, int TAPS>
 __global__ __launch_bounds__(CP_THREADS) void conv_prep_kernel(T* __restrict__ out, const T* __restrict__ x, int64_t x_ld, const float* __restrict__ conv_w, int taps_rt,
@@ -21,7 +49,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_prep_kernel(T* __restrict__ o
                                                                const int32_t* __restrict__ slots, const int32_t* __restrict__ pos0, const int32_t* __restrict__ len_after,
                                                                int n, int q_heads, int kv_heads, int dim, int vdim, int rows, int keep_first, int q_per, int v_per, int q_groups, int k_groups)
 {
-    extern __shared__ float smem[];                           // [R][channels of the group] | cos, sin [R][rot_dims / 2] each
+    extern __shared__ __attribute__((aligned(16))) float smem[];                           // [R][channels of the group] | cos, sin [R][rot_dims / 2] each
     const int taps = TAPS ? TAPS : taps_rt, keep = taps - 1;
     const int n0 = blockIdx.x * R, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const int nq = q_heads * dim, nk = kv_heads * dim, nv = kv_heads * vdim, C = nq + nk + nv;
@@ -49,8 +77,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_prep_kernel(T* __restrict__ o
             #pragma unroll
             for (int j = 0; j < (TAPS ? TAPS : 1); ++j)
             {
-                #pragma unroll
-                for (int e = 0; e < V; ++e) wt[j][e] = conv_w[(int64_t) j * C + ch + e];
+                load_f<V>(conv_w + (int64_t) j * C + ch, wt[j]);
             }
         }
         #pragma unroll
@@ -81,8 +108,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_prep_kernel(T* __restrict__ o
             if (keep > 0 && pos >= len_after[b] - keep) store_n<T, V>(rg + (int64_t) (pos % keep) * C, own);      // after this thread's own reads of the channel
             if (part < 2)
             {
-                #pragma unroll
-                for (int e = 0; e < V; ++e) smem[r * cols + i + e] = acc[e];
+                store_f<V>(smem + r * cols + i, acc);
                 continue;
             }
             store_n<T, V>(out + (int64_t) row * C + ch, acc);
@@ -121,8 +147,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_prep_kernel(T* __restrict__ o
         {
             const int row = n0 + r;
             float y[V];
-            #pragma unroll
-            for (int e = 0; e < V; ++e) y[e] = smem[r * cols + i + e];
+            load_f<V>(smem + r * cols + i, y);
             store_n<T, V>(out + (int64_t) row * C + c0 + i, y);
             if (part == 1)
             {
@@ -147,7 +172,7 @@ extern "C" int exl3_mix_conv_prep(void* out, const void* x, int64_t x_ld, const 
     if (n == 0) return EXL3_MIX_OK;
     const int vn = dtype == EXL3_MIX_BF16 ? 8 : 4;
     const bool vec = dim % vn == 0 && vdim % vn == 0 && x_ld % vn == 0 && (uintptr_t) x % 16 == 0 && (uintptr_t) out % 16 == 0 && (uintptr_t) conv_ring % 16 == 0 && (uintptr_t) ring_k % 16 == 0 &&
-                     (uintptr_t) ring_v % 16 == 0;
+                     (uintptr_t) ring_v % 16 == 0 && (uintptr_t) conv_w % 16 == 0;
     const bool many = vec && n >= 512;
     const int q_per = CP_CHANNELS / dim, v_per = CP_CHANNELS / vdim;
     const int q_groups = (q_heads + q_per - 1) / q_per, k_groups = (kv_heads + q_per - 1) / q_per, v_groups = (kv_heads + v_per - 1) / v_per;

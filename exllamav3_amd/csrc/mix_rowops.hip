@@ -24,8 +24,10 @@ __global__ __launch_bounds__(ROW_THREADS) void embed_copy_kernel(float* __restri
     }
 }
 
-// x[n] = table row of tokens[n] over its root mean square, times w; xc (optional): the same in the activation type
-template <typename T>
+// x[n] = table row of tokens[n] over its root mean square, times w; xc (optional): the same in the activation type.  V: elements per thread and access; the first
+// EN_HELD pieces of a thread stay in registers between the two passes.
+#define EN_HELD 4
+template <typename T, int V>
 __global__ __launch_bounds__(ROW_THREADS) void embed_norm_kernel(float* __restrict__ x, T* __restrict__ xc, int64_t xc_ld, const T* __restrict__ table,
                                                                  const int32_t* __restrict__ tokens, const float* __restrict__ w, float eps, int width, int vocab)
 {
@@ -34,15 +36,51 @@ __global__ __launch_bounds__(ROW_THREADS) void embed_norm_kernel(float* __restri
     int tok = tokens[n];
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
     const T* src = table + (int64_t) tok * width;
+    float held[EN_HELD][V];
     float ss = 0.f;
-    for (int i = threadIdx.x; i < width; i += ROW_THREADS) { const float v = to_f(src[i]); ss += v * v; }
+    #pragma unroll
+    for (int u = 0; u < EN_HELD; ++u)
+    {
+        const int i = (u * ROW_THREADS + threadIdx.x) * V;
+        #pragma unroll
+        for (int e = 0; e < V; ++e) held[u][e] = 0.f;
+        if (i < width) load_n<T, V>(src + i, held[u]);
+    }
+    #pragma unroll
+    for (int u = 0; u < EN_HELD; ++u)
+    {
+        #pragma unroll
+        for (int e = 0; e < V; ++e) ss += held[u][e] * held[u][e];
+    }
+    for (int i = (EN_HELD * ROW_THREADS + threadIdx.x) * V; i < width; i += ROW_THREADS * V)
+    {
+        float t[V];
+        load_n<T, V>(src + i, t);
+        #pragma unroll
+        for (int e = 0; e < V; ++e) ss += t[e] * t[e];
+    }
     ss = block_sum<ROW_WAVES>(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float) width + eps);
-    for (int i = threadIdx.x; i < width; i += ROW_THREADS)
+    auto write = [&](int i, float (&t)[V]) __attribute__((always_inline))
     {
-        const float v = to_f(src[i]) * inv * w[i];
-        x[(int64_t) n * width + i] = v;
-        if (xc) xc[(int64_t) n * xc_ld + i] = from_f<T>(v);
+        float wv[V];
+        load_n<float, V>(w + i, wv);
+        #pragma unroll
+        for (int e = 0; e < V; ++e) t[e] = t[e] * inv * wv[e];
+        store_n<float, V>(x + (int64_t) n * width + i, t);
+        if (xc) store_n<T, V>(xc + (int64_t) n * xc_ld + i, t);
+    };
+    #pragma unroll
+    for (int u = 0; u < EN_HELD; ++u)
+    {
+        const int i = (u * ROW_THREADS + threadIdx.x) * V;
+        if (i < width) write(i, held[u]);
+    }
+    for (int i = (EN_HELD * ROW_THREADS + threadIdx.x) * V; i < width; i += ROW_THREADS * V)
+    {
+        float t[V];
+        load_n<T, V>(src + i, t);
+        write(i, t);
     }
 }
 
@@ -444,7 +482,10 @@ extern "C" int exl3_mix_embed_norm(float* x, void* xc, int64_t xc_ld, const void
 {
     MIX_CHECK(x && table && tokens && w && n >= 0 && width > 0 && vocab > 0 && (!xc || xc_ld >= width), "mix_embed_norm: bad arguments");
     if (n == 0) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(embed_norm_kernel<T>, dim3(n), dim3(ROW_THREADS), 0, (hipStream_t) stream, x, (T*) xc, xc_ld, (const T*) table, tokens, w, eps, width, vocab));
+    const bool by4 = width % 4 == 0 && (uintptr_t) x % 16 == 0 && (uintptr_t) table % 16 == 0 && (uintptr_t) w % 16 == 0 && (!xc || (xc_ld % 4 == 0 && (uintptr_t) xc % 16 == 0));
+    #define EN_LAUNCH(VV) hipLaunchKernelGGL((embed_norm_kernel<T, VV>), dim3(n), dim3(ROW_THREADS), 0, (hipStream_t) stream, x, (T*) xc, xc_ld, (const T*) table, tokens, w, eps, width, vocab)
+    MIX_DISPATCH_T(dtype, if (by4) EN_LAUNCH(4); else EN_LAUNCH(1));
+    #undef EN_LAUNCH
     return mix_check_launch("mix_embed_norm");
 }
 

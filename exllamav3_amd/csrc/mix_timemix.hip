@@ -1,16 +1,16 @@
-// Time mixing with a decay per key channel and token and a bonus for the current token (RWKV-style).  Per head, with decays w_t in (0, 1] given by their logarithms:
+// Time mixing with a decay per key channel and token and a bonus for the current token (RWKV-style).  Per head, with decays w_t in (0, 1] given by their base-2 logarithms:
 //   o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,   S_t = diag(w_t) S_(t-1) + k_t v_t^T
 // Everything that enters the recurrence besides the projections is float32; the state [slot][head][dim][vdim] is float32.
 //
 //   token_shift    what the projections read: h + (h' - h) mu_m for every mix m, h' the previous token's row (of the step, or from the slot)
-//   decay_log      log w = -exp(w0 + W2 tanh(t)) from the low-rank input t, on the float32 matrix instruction
+//   decay_log2     log2 w = -log2(e) exp(w0 + W2 tanh(t)) from the low-rank input t
 //   timemix        prompt steps in tiles of 16 tokens, whole sequences or parallel segments; optionally with the head norm and gate that follow
 //   timemix_step   one row per sequence: decays, read-out, state update, head norm and gate in one launch
 //
-// A tile of 16 tokens is four products on the float32 matrix instruction.  With L_t the sum of the tile's log decays up to and including token t, L'_t the sum
-// before it and M = L_7 (the middle of the tile), q_t = r_t e^(L'_t - M) and p_t = k_t e^(M - L_t):
-//   S' = diag(e^M) S;   O = Q S' + A V,  A[t][j] = q_t . p_j for j < t, A[t][t] = sum_c r_t u k_t;   S <- diag(e^(L_15 - M)) (S' + P^T V)
-// Taking the exponents from the middle keeps both factors in range while every channel decays by less than e^-60 over each half of the tile; a tile with a
+// A tile of 16 tokens is four products on the float32 matrix instruction.  With L_t the sum of the tile's log2 decays up to and including token t, L'_t the sum
+// before it and M = L_7 (the middle of the tile), q_t = r_t 2^(L'_t - M) and p_t = k_t 2^(M - L_t):
+//   S' = diag(2^M) S;   O = Q S' + A V,  A[t][j] = q_t . p_j for j < t, A[t][t] = sum_c r_t u k_t;   S <- diag(2^(L_15 - M)) (S' + P^T V)
+// Taking the exponents from the middle keeps both factors in range while every channel decays by less than 2^-80 over each half of the tile; a tile with a
 // stronger decay (uniform over the workgroup) runs token by token on the same registers instead, in which every exponent is a decay's own.
 //
 // v_mfma_f32_16x16x4_f32: operand lane (g = lane / 16, c = lane % 16) holds row / column c and contraction slot g; result lane (g, c) holds rows 4g .. 4g+3 of column
@@ -27,7 +27,8 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 #define TM_WHOLE 0
 #define TM_SEG_LOCAL 1
 #define TM_SEG_FINAL 2
-#define TM_MAX_EXP 60.0f
+#define TM_MAX_EXP 80.0f
+#define TM_EXP2(x) __builtin_amdgcn_exp2f(x)
 
 // out[m][n] = h[n] + (h'[n] - h[n]) mu[m]; h' = the row before n in its sequence: the step's own where the sequence has it in the step, the slot's otherwise, zeros
 // ahead of the first token.  The last row of a sequence goes into its slot.  A thread holds V channels of R consecutive rows and of the row before them.
@@ -90,12 +91,75 @@ __global__ __launch_bounds__(256) void token_shift_kernel(T* __restrict__ out, c
     }
 }
 
-// out[n][c] = -exp(w0[c] + sum_r tanh(t[n][r]) w2[c][r]): 32 rows x 256 channels per workgroup, a wave takes 64 of the channels; tanh and the products are float32
+// out[n][c] = -log2(e) exp(w0[c] + sum_r tanh(t[n][r]) w2[c][r])
+__device__ __forceinline__ float decay_log2_f(float z) { return -1.4426950408889634f * expf(z); }
+
+// bfloat16 weights: a float32 factor is three bfloat16 pieces (8 + 8 + 8 bits of its 24), so three products on the bfloat16 matrix instruction are the float32 product
+// with an exact weight.  A wave takes 16 rows (their tanh is computed once, in registers) and 256 channels; weights come straight from memory as operands, 16 bytes per
+// lane.  The result tile is [channel][row]: a lane holds four neighbouring channels of one row.
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+#define DB_COLS 256
+#define DB_ROWS 64
+__global__ __launch_bounds__(256) void decay_log2_bf16_kernel(float* __restrict__ out, const bf16_t* __restrict__ t, int64_t t_ld, const bf16_t* __restrict__ w2,
+                                                              const float* __restrict__ w0, int n, int channels, int rank)
+{
+    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
+    const int n0 = blockIdx.x * DB_ROWS + w * 16, c0 = blockIdx.y * DB_COLS;
+    if (n0 >= n) return;
+    const bf16_t* tr = t + (int64_t) min(n0 + c, n - 1) * t_ld;       // rows beyond the last: computed and never stored
+    f32x4 acc[DB_COLS / 16];
+    #pragma unroll
+    for (int b = 0; b < DB_COLS / 16; ++b) acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < rank; k0 += 32)                             // rank is a multiple of 8: a lane's eight entries are all there or none
+    {
+        const int k = k0 + g * 8;
+        const bool ok = k < rank;
+        bf16x8 p0, p1, p2;
+        float f[8];
+        #pragma unroll
+        for (int e = 0; e < 8; ++e) f[e] = 0.f;
+        if (ok) load_n<bf16_t, 8>(tr + k, f);
+        #pragma unroll
+        for (int e = 0; e < 8; ++e)
+        {
+            const float y = tanhf(f[e]);
+            p0[e] = (__bf16) y;
+            const float y1 = y - (float) p0[e];
+            p1[e] = (__bf16) y1;
+            p2[e] = (__bf16) (y1 - (float) p1[e]);
+        }
+        #pragma unroll
+        for (int b = 0; b < DB_COLS / 16; ++b)
+        {
+            const int col = c0 + b * 16 + c;
+            union { bf16x8 v; uint4 x; } a;
+            a.x = (ok && col < channels) ? *(const uint4*) (w2 + (int64_t) col * rank + k) : uint4{0u, 0u, 0u, 0u};
+            acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, p2, acc[b], 0, 0, 0);
+            acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, p1, acc[b], 0, 0, 0);
+            acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, p0, acc[b], 0, 0, 0);
+        }
+    }
+    if (n0 + c >= n) return;
+    float* dst = out + (int64_t) (n0 + c) * channels;
+    #pragma unroll
+    for (int b = 0; b < DB_COLS / 16; ++b)
+    {
+        const int col = c0 + b * 16 + 4 * g;                          // channels is a multiple of 4
+        if (col >= channels) break;
+        float z[4], y[4];
+        load_n<float, 4>(w0 + col, z);
+        #pragma unroll
+        for (int i = 0; i < 4; ++i) y[i] = decay_log2_f(acc[b][i] + z[i]);
+        store_n<float, 4>(dst + col, y);
+    }
+}
+
+// Any sizes and float32 weights, on the float32 matrix instruction: 32 rows x 256 channels per workgroup, a wave takes 64 of the channels
 #define DL_ROWS 32
 #define DL_COLS 256
 #define DL_K 32
 template <typename T>
-__global__ __launch_bounds__(256) void decay_log_kernel(float* __restrict__ out, const T* __restrict__ t, int64_t t_ld, const T* __restrict__ w2, const float* __restrict__ w0, int n,
+__global__ __launch_bounds__(256) void decay_log2_kernel(float* __restrict__ out, const T* __restrict__ t, int64_t t_ld, const T* __restrict__ w2, const float* __restrict__ w0, int n,
                                                         int channels, int rank)
 {
     __shared__ __attribute__((aligned(16))) float ts[DL_ROWS * (DL_K + 4)];
@@ -157,31 +221,50 @@ __global__ __launch_bounds__(256) void decay_log_kernel(float* __restrict__ out,
             for (int i = 0; i < 4; ++i)
             {
                 const int row = n0 + a * 16 + 4 * g + i;
-                if (row < n) out[(int64_t) row * channels + col] = -expf(acc[a][b][i] + z0);
+                if (row < n) out[(int64_t) row * channels + col] = decay_log2_f(acc[a][b][i] + z0);
             }
         }
     }
 }
 
+// A loaded element that waits in a register of its own: 16-bit elements would be packed in pairs, and packing waits for the loads
+template <typename T> struct in_flight;
+template <> struct in_flight<bf16_t>
+{
+    uint32_t u;
+    __device__ __forceinline__ void load(const bf16_t* p) { u = p->u; }
+    __device__ __forceinline__ float value() const { return __uint_as_float(u << 16); }
+    __device__ __forceinline__ void arrive() { asm volatile("" : "+v"(u)); }
+};
+template <> struct in_flight<float>
+{
+    float f;
+    __device__ __forceinline__ void load(const float* p) { f = *p; }
+    __device__ __forceinline__ float value() const { return f; }
+    __device__ __forceinline__ void arrive() { asm volatile("" : "+v"(f)); }
+};
+
 // DT: 16-row blocks of the (zero-padded) key dim.  Preparation: wave w owns the tile's tokens 4w .. 4w + 3, lane l the channels l, l + 64, ...
-// out (optional, vdim <= 64): the heads after norm and gate, o / rms(o) * norm_w * silu(gate), instead of o.
-template <typename T, int DT, int MODE>
-__global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __restrict__ o, T* __restrict__ out, int64_t out_ld, const T* __restrict__ gate, int64_t gate_ld,
+// FUSED (vdim <= 64): out receives the heads after norm and gate, o / rms(o) * norm_w * silu(gate), instead of o.
+template <typename T, int DT, int MODE, bool FUSED>
+__global__ __launch_bounds__(TM_THREADS, DT <= 4 ? 3 : (DT <= 8 ? 2 : 1)) void timemix_chunk_kernel(float* __restrict__ o, T* __restrict__ out, int64_t out_ld, const T* __restrict__ gate, int64_t gate_ld,
                                                                    const float* __restrict__ norm_w, float eps, float* __restrict__ state,
                                                                    const T* __restrict__ r, int64_t r_ld, const T* __restrict__ k, int64_t k_ld, const T* __restrict__ v, int64_t v_ld,
-                                                                   const float* __restrict__ logw, const float* __restrict__ u, const int32_t* __restrict__ cu,
+                                                                   const float* __restrict__ log2w, const float* __restrict__ u, const int32_t* __restrict__ cu,
                                                                    const int32_t* __restrict__ slots, const int32_t* __restrict__ pos0, int heads, int dim, int vdim,
                                                                    int segs, int seg_len, float* __restrict__ seg_state, float* __restrict__ seg_decay)
 {
     constexpr int DP = DT * 16, LS = DP + 4, CI = (DP + 63) / 64, PS = TM_TILE + 4, TW = TM_TILE / TM_WAVES;
+    static_assert(TW == 4, "a wave prepares four tokens, a lane holds the values of four");
     constexpr bool READ = MODE != TM_SEG_LOCAL;
-    __shared__ __attribute__((aligned(16))) float ks[TM_TILE * LS], ws[TM_TILE * LS];
+    constexpr int WP = READ && TM_WAVES * PS > LS ? TM_TILE * TM_WAVES * PS : TM_TILE * LS;
+    __shared__ __attribute__((aligned(16))) float ks[TM_TILE * LS], ws[WP];
     __shared__ __attribute__((aligned(16))) float rs[READ ? TM_TILE * LS : 4];
-    __shared__ __attribute__((aligned(16))) float ps[READ ? TM_WAVES * TM_TILE * PS : 4];
+    float* const ps = ws;                                             // a tile needs either its decays one by one or the partial scores
     __shared__ __attribute__((aligned(16))) float em[DP], et[DP];
-    __shared__ float tot[2][TM_WAVES][CI * 64], dg[2][TM_TILE], red[TM_WAVES][TM_TILE];
+    __shared__ __attribute__((aligned(16))) float dg[2][TM_TILE][4], tot[2][TM_WAVES][CI * 64], red[TM_WAVES][TM_TILE];
     const int b = (MODE == TM_WHOLE) ? blockIdx.x : blockIdx.x / segs, h = blockIdx.y;
-    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
+    const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
     const int col = blockIdx.z * TM_COLS + w * 16 + c;
     const bool col_ok = col < vdim;
     int first = cu[b], last = cu[b + 1];
@@ -213,32 +296,41 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
         uc[ci] = (READ && lane + 64 * ci < dim) ? u[h * dim + lane + 64 * ci] : 0.f;
         seg_sum[ci] = 0.f;
     }
-    // the rows of the next tile wait in registers, as loaded, while the current one is computed
-    T tr[CI][TW], tk[CI][TW], tv[4];
-    float tw[CI][TW];
-    const T zero = from_f<T>(0.f);
+    // The rows of the next tile wait in registers, as loaded, while the current one is computed.  Nothing is conditional: places beyond the tile, the key dim or the value
+    // dim read their nearest neighbour; where the value matters (k and the decays) it is replaced when it is used.
+    in_flight<T> tr[CI][TW], tk[CI][TW], tv[4], tg[4];
+    in_flight<float> tw[CI][TW];
+    int chc[CI];
+    #pragma unroll
+    for (int ci = 0; ci < CI; ++ci) chc[ci] = min(lane + 64 * ci, dim - 1);
+    const int colc = min(col, vdim - 1);
+    const float inv_vdim = 1.0f / (float) vdim;
+    const float nw = FUSED ? norm_w[h * vdim + colc] : 0.f;
     auto fetch = [&](int n0) __attribute__((always_inline))
     {
         #pragma unroll
         for (int j = 0; j < TW; ++j)
         {
-            const int t = n0 + w * TW + j;
+            const int t = min(n0 + w * TW + j, last - 1);             // the same for the whole wave: a lane adds its channel to a scalar address
+            const T* kr = k + (int64_t) t * k_ld + h * dim;
+            const T* rr = r + (int64_t) t * r_ld + h * dim;
+            const float* wr = log2w + ((int64_t) t * heads + h) * dim;
             #pragma unroll
             for (int ci = 0; ci < CI; ++ci)
             {
-                const int ch = lane + 64 * ci;
-                const bool ok = t < last && ch < dim;
-                const int64_t at = (int64_t) h * dim + ch;
-                tk[ci][j] = ok ? k[(int64_t) t * k_ld + at] : zero;
-                tr[ci][j] = (READ && ok) ? r[(int64_t) t * r_ld + at] : zero;
-                tw[ci][j] = ok ? logw[(int64_t) t * heads * dim + at] : 0.f;
+                tk[ci][j].load(kr + chc[ci]);
+                tw[ci][j].load(wr + chc[ci]);
+                if (READ) tr[ci][j].load(rr + chc[ci]);
             }
         }
+        const T* vb = v + (int64_t) n0 * v_ld + h * vdim;
+        const T* gb = FUSED ? gate + (int64_t) n0 * gate_ld + h * vdim : nullptr;
         #pragma unroll
         for (int i = 0; i < 4; ++i)
         {
-            const int t = n0 + 4 * g + i;
-            tv[i] = (t < last && col_ok) ? v[(int64_t) t * v_ld + (int64_t) h * vdim + col] : zero;
+            const int t = min(4 * g + i, last - 1 - n0);
+            tv[i].load(vb + t * (int) v_ld + colc);
+            if (FUSED) tg[i].load(gb + t * (int) gate_ld + colc);
         }
     };
     fetch(first);
@@ -246,10 +338,11 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
     for (int n0 = first; n0 < last; n0 += TM_TILE, par ^= 1)
     {
         const int tc = min(TM_TILE, last - n0);
-        float kf[CI][TW], rf[CI][TW], lw[CI][TW], vr[4];
+        float vr[4], gr[4];
         float bonus[TW];
         #pragma unroll
         for (int j = 0; j < TW; ++j) bonus[j] = 0.f;
+        float kf[CI][TW];
         #pragma unroll
         for (int ci = 0; ci < CI; ++ci)
         {
@@ -257,25 +350,30 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
             #pragma unroll
             for (int j = 0; j < TW; ++j)
             {
-                kf[ci][j] = to_f(tk[ci][j]); rf[ci][j] = to_f(tr[ci][j]); lw[ci][j] = tw[ci][j];
-                sum += lw[ci][j];
-                bonus[j] += rf[ci][j] * uc[ci] * kf[ci][j];
+                const bool ok = w * TW + j < tc && lane + 64 * ci < dim;
+                kf[ci][j] = ok ? tk[ci][j].value() : 0.f;
+                tw[ci][j].f = ok ? tw[ci][j].f : 0.f;
+                sum += tw[ci][j].f;
+                if (READ) bonus[j] = __builtin_fmaf(tr[ci][j].value() * uc[ci], kf[ci][j], bonus[j]);
             }
             tot[par][w][lane + 64 * ci] = sum;
         }
         #pragma unroll
-        for (int i = 0; i < 4; ++i) vr[i] = to_f(tv[i]);
+        for (int i = 0; i < 4; ++i)
+        {
+            vr[i] = tv[i].value();
+            if (FUSED) { const float z = tg[i].value(); gr[i] = z * nw * __builtin_amdgcn_rcpf(1.0f + TM_EXP2(z * -1.4426950408889634f)); }
+        }
         if (READ)
         {
             #pragma unroll
             for (int j = 0; j < TW; ++j)
             {
-                const float s = wave_sum(bonus[j]);
-                if (lane == 0) dg[par][w * TW + j] = s;
+                const float s = row16_sum(bonus[j]);
+                if (c == 0) dg[par][w * TW + j][g] = s;
             }
         }
         __syncthreads();                                              // tot and dg are there; the previous tile's reads of everything else are over
-        if (n0 + TM_TILE < last) fetch(n0 + TM_TILE);
         bool strong = false;
         float half0[CI], half1[CI], base[CI];
         #pragma unroll
@@ -302,50 +400,56 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
                     const int at = (w * TW + j) * LS + ch;
                     if (slow)
                     {
-                        if (READ) rs[at] = rf[ci][j];
+                        if (READ) rs[at] = tr[ci][j].value();
                         ks[at] = kf[ci][j];
-                        ws[at] = expf(lw[ci][j]);
+                        ws[at] = TM_EXP2(tw[ci][j].f);
                     }
                     else
                     {
-                        if (READ) rs[at] = rf[ci][j] * expf(e);
-                        e += lw[ci][j];
-                        ks[at] = kf[ci][j] * expf(-e);
+                        if (READ) rs[at] = tr[ci][j].value() * TM_EXP2(e);
+                        e += tw[ci][j].f;
+                        ks[at] = kf[ci][j] * TM_EXP2(-e);
                     }
                 }
-                if (w == 0) em[ch] = expf(half0[ci]);
-                if (w == 3) et[ch] = expf(half1[ci]);
+                if (w == 0) em[ch] = TM_EXP2(half0[ci]);
+                if (w == 3) et[ch] = TM_EXP2(half1[ci]);
             }
         }
         __syncthreads();
+        if (n0 + TM_TILE < last) fetch(n0 + TM_TILE);                 // under the tile's matrix work
         f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
         if (slow)
         {
-            #pragma unroll
-            for (int t = 0; t < TM_TILE; ++t)
+            #pragma unroll 1                                          // rolled: the rare path must not cost the other one registers
+            for (int t = 0; t < tc; ++t)
             {
-                if (t >= tc) break;
-                const float vv = __shfl(vr[t & 3], (t >> 2) * 16 + c, 64);
+                const int tg4 = t >> 2, ti = t & 3;
+                const float own = ti == 0 ? vr[0] : (ti == 1 ? vr[1] : (ti == 2 ? vr[2] : vr[3]));
+                const float vv = __shfl(own, tg4 * 16 + c, 64);
                 float po = 0.f;
                 #pragma unroll
                 for (int kt = 0; kt < DT; ++kt)
                 {
                     const int at = t * LS + kt * 16 + 4 * g;
-                    const f32x4 kk = *(const f32x4*) (ks + at), dd = *(const f32x4*) (ws + at);
                     if (READ)
                     {
                         const f32x4 rr = *(const f32x4*) (rs + at);
                         #pragma unroll
                         for (int i = 0; i < 4; ++i) po = __builtin_fmaf(rr[i], S[kt][i], po);
                     }
+                    const f32x4 kk = *(const f32x4*) (ks + at), dd = *(const f32x4*) (ws + at);
                     #pragma unroll
                     for (int i = 0; i < 4; ++i) S[kt][i] = __builtin_fmaf(dd[i], S[kt][i], kk[i] * vv);
+                    __builtin_amdgcn_sched_barrier(0);
                 }
                 if (READ)
                 {
                     po += __shfl_xor(po, 16, 64);
                     po += __shfl_xor(po, 32, 64);
-                    if (g == (t >> 2)) acc[t & 3] = __builtin_fmaf(dg[par][t], vv, po);
+                    const f32x4 o4 = *(const f32x4*) dg[par][t];
+                    po = __builtin_fmaf((o4[0] + o4[1]) + (o4[2] + o4[3]), vv, po);
+                    #pragma unroll
+                    for (int i = 0; i < 4; ++i) acc[i] = (g == tg4 && ti == i) ? po : acc[i];
                 }
             }
         }
@@ -358,15 +462,18 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
                 // the scores' contraction is shared out over the waves; partial tiles meet in LDS
                 f32x4 sc = f32x4{0.f, 0.f, 0.f, 0.f};
                 #pragma unroll
+                for (int m = 0; m < (DT + TM_WAVES - 1) / TM_WAVES; ++m)
+                {
+                    const int kt = w + TM_WAVES * m;
+                    if (DT % TM_WAVES != 0 && kt >= DT) break;        // uniform for the wave
+                    const f32x4 a = *(const f32x4*) (rs + c * LS + kt * 16 + 4 * g), bk = *(const f32x4*) (ks + c * LS + kt * 16 + 4 * g);
+                    #pragma unroll
+                    for (int i = 0; i < 4; ++i) sc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], bk[i], sc, 0, 0, 0);
+                }
+                #pragma unroll
                 for (int kt = 0; kt < DT; ++kt)
                 {
                     const f32x4 a = *(const f32x4*) (rs + c * LS + kt * 16 + 4 * g);
-                    if ((kt & (TM_WAVES - 1)) == w)
-                    {
-                        const f32x4 bk = *(const f32x4*) (ks + c * LS + kt * 16 + 4 * g);
-                        #pragma unroll
-                        for (int i = 0; i < 4; ++i) sc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], bk[i], sc, 0, 0, 0);
-                    }
                     #pragma unroll
                     for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], S[kt][i], acc, 0, 0, 0);
                 }
@@ -376,7 +483,8 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
                 f32x4 a = *(const f32x4*) (ps + c * PS + 4 * g);
                 #pragma unroll
                 for (int ww = 1; ww < TM_WAVES; ++ww) a += *(const f32x4*) (ps + (ww * TM_TILE + c) * PS + 4 * g);
-                const float own = dg[par][c];
+                const f32x4 o4 = *(const f32x4*) dg[par][c];
+                const float own = (o4[0] + o4[1]) + (o4[2] + o4[3]);
                 #pragma unroll
                 for (int i = 0; i < 4; ++i)
                 {
@@ -394,7 +502,16 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
             for (int kt = 0; kt < DT; ++kt) S[kt] *= *(const f32x4*) (et + kt * 16 + 4 * g);
         }
         if (!READ) continue;
-        if (out)
+        // the next tile's rows have had the matrix work's time to arrive; waiting for them here, ahead of this tile's stores, keeps the stores out of that wait
+        #pragma unroll
+        for (int j = 0; j < TW; ++j)
+        {
+            #pragma unroll
+            for (int ci = 0; ci < CI; ++ci) { tk[ci][j].arrive(); tr[ci][j].arrive(); tw[ci][j].arrive(); }
+            tv[j].arrive();
+            if (FUSED) tg[j].arrive();
+        }
+        if (FUSED)
         {
             #pragma unroll
             for (int i = 0; i < 4; ++i)
@@ -403,21 +520,20 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
                 if (c == 0) red[w][4 * g + i] = s;
             }
             __syncthreads();
+            const f32x4 ss = (*(const f32x4*) (red[0] + 4 * g) + *(const f32x4*) (red[1] + 4 * g)) + (*(const f32x4*) (red[2] + 4 * g) + *(const f32x4*) (red[3] + 4 * g));
+            T* ob = out + (int64_t) n0 * out_ld + h * vdim;
+            #pragma unroll
+            for (int i = 0; i < 4; ++i)
+            {
+                const float y = acc[i] * __builtin_amdgcn_rsqf(ss[i] * inv_vdim + eps) * gr[i];
+                if (4 * g + i < tc && col_ok) ob[(4 * g + i) * (int) out_ld + col] = from_f<T>(y);
+            }
+            continue;
         }
+        float* ob = o + ((int64_t) n0 * heads + h) * vdim;
         #pragma unroll
         for (int i = 0; i < 4; ++i)
-        {
-            const int t = 4 * g + i;
-            if (t >= tc || !col_ok) continue;
-            if (out)
-            {
-                const float ss = (red[0][t] + red[1][t]) + (red[2][t] + red[3][t]);
-                const float inv = 1.0f / sqrtf(ss / (float) vdim + eps);
-                const int64_t at = (int64_t) h * vdim + col;
-                out[(int64_t) (n0 + t) * out_ld + at] = from_f<T>(acc[i] * inv * norm_w[at] * silu_f(to_f(gate[(int64_t) (n0 + t) * gate_ld + at])));
-            }
-            else o[((int64_t) (n0 + t) * heads + h) * vdim + col] = acc[i];
-        }
+            if (4 * g + i < tc && col_ok) ob[(4 * g + i) * heads * vdim + col] = acc[i];
     }
     if (MODE == TM_SEG_FINAL) return;
     #pragma unroll
@@ -436,7 +552,7 @@ __global__ __launch_bounds__(TM_THREADS) void timemix_chunk_kernel(float* __rest
         for (int ci = 0; ci < CI; ++ci)
         {
             const int ch = lane + 64 * ci;
-            if (ch < dim) seg_decay[((int64_t) blockIdx.x * heads + h) * dim + ch] = expf(seg_sum[ci]);
+            if (ch < dim) seg_decay[((int64_t) blockIdx.x * heads + h) * dim + ch] = TM_EXP2(seg_sum[ci]);
         }
     }
 }
@@ -484,7 +600,7 @@ __global__ __launch_bounds__(TS_THREADS) void timemix_step_kernel(T* __restrict_
                                                                   const T* __restrict__ k, int64_t k_ld, const T* __restrict__ v, int64_t v_ld, const T* __restrict__ gate, int64_t gate_ld,
                                                                   const T* __restrict__ t, int64_t t_ld, const T* __restrict__ w2, const float* __restrict__ w0,
                                                                   const float* __restrict__ u, const float* __restrict__ norm_w, const int32_t* __restrict__ tok_pos,
-                                                                  const int32_t* __restrict__ slots, int heads, int dim, int vdim, int rank, float eps)
+                                                                  const int32_t* __restrict__ slots, int heads, int dim, int vdim, int rank, float eps, int w_vec)
 {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     __shared__ float red[TS_THREADS / 64];
@@ -497,6 +613,20 @@ __global__ __launch_bounds__(TS_THREADS) void timemix_step_kernel(T* __restrict_
     float* ub = dc + dim;                                             // [dim] r u k
     float* th = ub + dim;                                             // [rank] tanh of the low-rank input
     const int n = blockIdx.x, h = blockIdx.y;
+    const int sub = threadIdx.x & 7, ch0 = threadIdx.x >> 3;
+    const int r0 = threadIdx.x / cg, c0 = (threadIdx.x - r0 * cg) * V;
+    const bool live = r0 < rp, resume = tok_pos[n] > 0;
+    float* st = state + ((int64_t) slots[n] * heads + h) * dim * vdim;
+    // what the first pass of each loop below needs is on its way before the first barrier: eight entries of a channel's weights, two pieces of the state
+    float wreg[8], held[2][V];
+    if (w_vec && ch0 < dim && sub * 8 < rank) load_n<T, 8>(w2 + ((int64_t) h * dim + ch0) * rank + sub * 8, wreg);
+    #pragma unroll
+    for (int x = 0; x < 2; ++x)
+    {
+        #pragma unroll
+        for (int e = 0; e < V; ++e) held[x][e] = 0.f;
+        if (live && resume && r0 + x * rp < dim) load_n<float, V>(st + (int64_t) (r0 + x * rp) * vdim + c0, held[x]);
+    }
     for (int i = threadIdx.x; i < dim; i += TS_THREADS)
     {
         const int64_t at = (int64_t) h * dim + i;
@@ -504,39 +634,36 @@ __global__ __launch_bounds__(TS_THREADS) void timemix_step_kernel(T* __restrict_
         rk[i] = a; kk[i] = b; ub[i] = a * u[at] * b;
     }
     for (int i = threadIdx.x; i < rank; i += TS_THREADS) th[i] = tanhf(to_f(t[(int64_t) n * t_ld + i]));
-    const int r0 = threadIdx.x / cg, c0 = (threadIdx.x - r0 * cg) * V;
-    const bool live = r0 < rp, resume = tok_pos[n] > 0;
-    float* st = state + ((int64_t) slots[n] * heads + h) * dim * vdim;
     __syncthreads();
+    for (int i0 = 0; i0 < dim; i0 += TS_THREADS / 8)                  // uniform trip count: the shuffles see whole groups of eight
     {
-        const int sub = threadIdx.x & 7;
-        for (int i0 = 0; i0 < dim; i0 += TS_THREADS / 8)              // uniform trip count: the shuffles see whole groups of eight
+        const int i = i0 + ch0;
+        float z = 0.f;
+        if (i < dim)
         {
-            const int i = i0 + (threadIdx.x >> 3);
-            float z = 0.f;
-            if (i < dim)
+            const T* wr = w2 + ((int64_t) h * dim + i) * rank;
+            if (w_vec)
             {
-                const T* wr = w2 + ((int64_t) h * dim + i) * rank;
-                for (int x = sub; x < rank; x += 8) z = __builtin_fmaf(th[x], to_f(wr[x]), z);
+                for (int x = sub * 8; x < rank; x += 64)
+                {
+                    if (i0 > 0 || x >= 64) load_n<T, 8>(wr + x, wreg);
+                    #pragma unroll
+                    for (int e = 0; e < 8; ++e) z = __builtin_fmaf(th[x + e], wreg[e], z);
+                }
             }
-            z += __shfl_xor(z, 1, 64); z += __shfl_xor(z, 2, 64); z += __shfl_xor(z, 4, 64);
-            if (i < dim && sub == 0) dc[i] = expf(-expf(z + w0[(int64_t) h * dim + i]));
+            else for (int x = sub; x < rank; x += 8) z = __builtin_fmaf(th[x], to_f(wr[x]), z);
         }
+        z += __shfl_xor(z, 1, 64); z += __shfl_xor(z, 2, 64); z += __shfl_xor(z, 4, 64);
+        if (i < dim && sub == 0) dc[i] = expf(-expf(z + w0[(int64_t) h * dim + i]));
     }
     __syncthreads();
     if (live)
     {
-        const T* vp = v + (int64_t) n * v_ld + (int64_t) h * vdim + c0;
         float vv[V], acc[V];
         #pragma unroll
-        for (int e = 0; e < V; ++e) { vv[e] = to_f(vp[e]); acc[e] = 0.f; }
-        #pragma unroll 4
-        for (int row = r0; row < dim; row += rp)
+        for (int e = 0; e < V; ++e) { vv[e] = to_f(v[(int64_t) n * v_ld + (int64_t) h * vdim + c0 + e]); acc[e] = 0.f; }
+        auto visit = [&](int row, float (&s)[V]) __attribute__((always_inline))
         {
-            float* sp = st + (int64_t) row * vdim + c0;
-            float s[V];
-            if constexpr (V == 4) { const float4 q = resume ? *(const float4*) sp : make_float4(0.f, 0.f, 0.f, 0.f); s[0] = q.x; s[1] = q.y; s[2] = q.z; s[V - 1] = q.w; }
-            else s[0] = resume ? sp[0] : 0.f;
             const float kx = kk[row], rx = rk[row], dx = dc[row], ux = ub[row];
             #pragma unroll
             for (int e = 0; e < V; ++e)
@@ -544,7 +671,19 @@ __global__ __launch_bounds__(TS_THREADS) void timemix_step_kernel(T* __restrict_
                 acc[e] = __builtin_fmaf(rx, s[e], __builtin_fmaf(ux, vv[e], acc[e]));
                 s[e] = __builtin_fmaf(dx, s[e], kx * vv[e]);
             }
-            if constexpr (V == 4) *(float4*) sp = make_float4(s[0], s[1], s[2], s[V - 1]); else sp[0] = s[0];
+            store_n<float, V>(st + (int64_t) row * vdim + c0, s);
+        };
+        #pragma unroll
+        for (int x = 0; x < 2; ++x)
+            if (r0 + x * rp < dim) visit(r0 + x * rp, held[x]);
+        #pragma unroll 4
+        for (int row = r0 + 2 * rp; row < dim; row += rp)
+        {
+            float s[V];
+            #pragma unroll
+            for (int e = 0; e < V; ++e) s[e] = 0.f;
+            if (resume) load_n<float, V>(st + (int64_t) row * vdim + c0, s);
+            visit(row, s);
         }
         #pragma unroll
         for (int e = 0; e < V; ++e) part[r0 * vdim + c0 + e] = acc[e];
@@ -592,13 +731,19 @@ extern "C" int exl3_mix_token_shift(void* out, const void* h, int64_t h_ld, void
     return mix_check_launch("mix_token_shift");
 }
 
-extern "C" int exl3_mix_decay_log(float* out, const void* t, int64_t t_ld, const void* w2, const float* w0, int n, int channels, int rank, int dtype, void* stream)
+extern "C" int exl3_mix_decay_log2(float* out, const void* t, int64_t t_ld, const void* w2, const float* w0, int n, int channels, int rank, int dtype, void* stream)
 {
-    MIX_CHECK(out && t && w2 && w0 && n >= 0 && channels > 0 && rank > 0 && t_ld >= rank && (channels + DL_COLS - 1) / DL_COLS <= 65535, "mix_decay_log: bad arguments");
+    MIX_CHECK(out && t && w2 && w0 && n >= 0 && channels > 0 && rank > 0 && t_ld >= rank && (channels + DL_COLS - 1) / DL_COLS <= 65535, "mix_decay_log2: bad arguments");
     if (n == 0) return EXL3_MIX_OK;
-    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(decay_log_kernel<T>, dim3((n + DL_ROWS - 1) / DL_ROWS, (channels + DL_COLS - 1) / DL_COLS), dim3(256), 0, (hipStream_t) stream, out, (const T*) t,
+    if (dtype == EXL3_MIX_BF16 && rank % 8 == 0 && t_ld % 8 == 0 && channels % 4 == 0 && (uintptr_t) t % 16 == 0 && (uintptr_t) w2 % 16 == 0 && (uintptr_t) w0 % 16 == 0 && (uintptr_t) out % 16 == 0)
+    {
+        hipLaunchKernelGGL(decay_log2_bf16_kernel, dim3((n + DB_ROWS - 1) / DB_ROWS, (channels + DB_COLS - 1) / DB_COLS), dim3(256), 0, (hipStream_t) stream, out, (const bf16_t*) t, t_ld,
+                           (const bf16_t*) w2, w0, n, channels, rank);
+        return mix_check_launch("mix_decay_log2");
+    }
+    MIX_DISPATCH_T(dtype, hipLaunchKernelGGL(decay_log2_kernel<T>, dim3((n + DL_ROWS - 1) / DL_ROWS, (channels + DL_COLS - 1) / DL_COLS), dim3(256), 0, (hipStream_t) stream, out, (const T*) t,
                                              t_ld, (const T*) w2, w0, n, channels, rank));
-    return mix_check_launch("mix_decay_log");
+    return mix_check_launch("mix_decay_log2");
 }
 
 static int timemix_check(const char* what, int heads, int dim, int vdim)
@@ -609,30 +754,32 @@ static int timemix_check(const char* what, int heads, int dim, int vdim)
 
 template <int MODEV>
 static int timemix_launch(float* o, void* out, int64_t out_ld, const void* gate, int64_t gate_ld, const float* norm_w, float eps, float* state, const void* r, int64_t r_ld, const void* k,
-                          int64_t k_ld, const void* v, int64_t v_ld, const float* logw, const float* u, const int32_t* cu, const int32_t* slots, const int32_t* pos0, int batch, int heads,
+                          int64_t k_ld, const void* v, int64_t v_ld, const float* log2w, const float* u, const int32_t* cu, const int32_t* slots, const int32_t* pos0, int batch, int heads,
                           int dim, int vdim, int segs, int seg_len, float* seg_state, float* seg_decay, int dtype, void* stream)
 {
     const dim3 grid(batch * segs, heads, (vdim + TM_COLS - 1) / TM_COLS);
-    #define TM_LAUNCH(DTV) hipLaunchKernelGGL((timemix_chunk_kernel<T, DTV, MODEV>), grid, dim3(TM_THREADS), 0, (hipStream_t) stream, o, (T*) out, out_ld, (const T*) gate, gate_ld, norm_w, \
-                                              eps, state, (const T*) r, r_ld, (const T*) k, k_ld, (const T*) v, v_ld, logw, u, cu, slots, pos0, heads, dim, vdim, segs, seg_len, seg_state, \
+    #define TM_LAUNCH_F(DTV, FV) hipLaunchKernelGGL((timemix_chunk_kernel<T, DTV, MODEV, FV>), grid, dim3(TM_THREADS), 0, (hipStream_t) stream, o, (T*) out, out_ld, (const T*) gate, gate_ld, norm_w, \
+                                              eps, state, (const T*) r, r_ld, (const T*) k, k_ld, (const T*) v, v_ld, log2w, u, cu, slots, pos0, heads, dim, vdim, segs, seg_len, seg_state, \
                                               seg_decay)
+    #define TM_LAUNCH(DTV) do { if (MODEV != TM_SEG_LOCAL && out) TM_LAUNCH_F(DTV, (MODEV != TM_SEG_LOCAL)); else TM_LAUNCH_F(DTV, false); } while (0)
     MIX_DISPATCH_T(dtype, if (dim <= 32) TM_LAUNCH(2); else if (dim <= 48) TM_LAUNCH(3); else if (dim <= 64) TM_LAUNCH(4); else if (dim <= 128) TM_LAUNCH(8); else TM_LAUNCH(16));
     #undef TM_LAUNCH
+    #undef TM_LAUNCH_F
     return mix_check_launch("mix_timemix");
 }
 
 extern "C" int exl3_mix_timemix(float* o, void* out, int64_t out_ld, const void* gate, int64_t gate_ld, const float* norm_w, float eps, float* state, const void* r, int64_t r_ld,
-                                const void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* logw, const float* u, const int32_t* cu, const int32_t* slots,
+                                const void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* log2w, const float* u, const int32_t* cu, const int32_t* slots,
                                 const int32_t* pos0, int batch, int heads, int dim, int vdim, int segs, int seg_len, float* seg_state, float* seg_decay, int dtype, void* stream)
 {
-    MIX_CHECK((o || out) && state && r && k && v && logw && u && cu && slots && pos0 && batch >= 0, "mix_timemix: null pointer");
+    MIX_CHECK((o || out) && state && r && k && v && log2w && u && cu && slots && pos0 && batch >= 0, "mix_timemix: null pointer");
     if (int rc = timemix_check("mix_timemix", heads, dim, vdim)) return rc;
-    MIX_CHECK(r_ld >= (int64_t) heads * dim && k_ld >= (int64_t) heads * dim && v_ld >= (int64_t) heads * vdim, "mix_timemix: bad row strides");
-    MIX_CHECK(!out || (gate && norm_w && vdim <= TM_COLS && out_ld >= (int64_t) heads * vdim && gate_ld >= (int64_t) heads * vdim),
+    MIX_CHECK(r_ld >= (int64_t) heads * dim && k_ld >= (int64_t) heads * dim && v_ld >= (int64_t) heads * vdim && v_ld <= (1 << 26), "mix_timemix: bad row strides");
+    MIX_CHECK(!out || (gate && norm_w && vdim <= TM_COLS && out_ld >= (int64_t) heads * vdim && gate_ld >= (int64_t) heads * vdim && gate_ld <= (1 << 26) && out_ld <= (1 << 26)),
               "mix_timemix: norm and gate in the same launch need vdim <= %d, the gate and the weight", TM_COLS);
     MIX_CHECK(segs >= 1 && (segs == 1 || (seg_len >= 1 && seg_state && seg_decay)), "mix_timemix: bad segment arguments");
     if (batch == 0) return EXL3_MIX_OK;
-    #define TM_ARGS o, out, out_ld, gate, gate_ld, norm_w, eps, state, r, r_ld, k, k_ld, v, v_ld, logw, u, cu, slots, pos0, batch, heads, dim, vdim, segs, seg_len, seg_state, seg_decay, dtype, stream
+    #define TM_ARGS o, out, out_ld, gate, gate_ld, norm_w, eps, state, r, r_ld, k, k_ld, v, v_ld, log2w, u, cu, slots, pos0, batch, heads, dim, vdim, segs, seg_len, seg_state, seg_decay, dtype, stream
     if (segs == 1) return timemix_launch<TM_WHOLE>(TM_ARGS);
     int rc = timemix_launch<TM_SEG_LOCAL>(TM_ARGS);
     if (rc) return rc;
@@ -645,8 +792,8 @@ extern "C" int exl3_mix_timemix(float* o, void* out, int64_t out_ld, const void*
 }
 
 extern "C" int exl3_mix_timemix_step(void* out, int64_t out_ld, float* state, const void* r, int64_t r_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, const void* gate,
-                                     int64_t gate_ld, const void* t, int64_t t_ld, const void* w2, const float* w0, const float* u, const float* norm_w, const int32_t* tok_pos,
-                                     const int32_t* slots, int n, int heads, int dim, int vdim, int rank, float eps, int dtype, void* stream)
+                                     int64_t gate_ld, const void* t, int64_t t_ld, const void* w2, const float* w0, const float* u, const float* norm_w, const int32_t* tok_pos, const int32_t* slots, int n,
+                                     int heads, int dim, int vdim, int rank, float eps, int dtype, void* stream)
 {
     MIX_CHECK(out && state && r && k && v && gate && t && w2 && w0 && u && norm_w && tok_pos && slots && n >= 0, "mix_timemix_step: null pointer");
     if (int rc = timemix_check("mix_timemix_step", heads, dim, vdim)) return rc;
@@ -654,11 +801,12 @@ extern "C" int exl3_mix_timemix_step(void* out, int64_t out_ld, float* state, co
               rank > 0 && rank <= 4096 && t_ld >= rank, "mix_timemix_step: bad row strides or rank %d (<= 4096)", rank);
     if (n == 0) return EXL3_MIX_OK;
     const bool by4 = vdim % 4 == 0 && (uintptr_t) state % 16 == 0;
+    const int w_vec = rank % 8 == 0 && (uintptr_t) w2 % 16 == 0;
     MIX_CHECK(by4 || vdim <= TS_THREADS, "mix_timemix_step: vdim %d must be a multiple of 4 or at most %d", vdim, TS_THREADS);
     const int cg = by4 ? vdim / 4 : vdim;
     const size_t sm = ((size_t) (TS_THREADS / cg) * vdim + 4 * dim + rank) * sizeof(float);
     #define TS_LAUNCH(VV) hipLaunchKernelGGL((timemix_step_kernel<T, VV>), dim3(n, heads), dim3(TS_THREADS), sm, (hipStream_t) stream, (T*) out, out_ld, state, (const T*) r, r_ld, (const T*) k, \
-                                             k_ld, (const T*) v, v_ld, (const T*) gate, gate_ld, (const T*) t, t_ld, (const T*) w2, w0, u, norm_w, tok_pos, slots, heads, dim, vdim, rank, eps)
+                                             k_ld, (const T*) v, v_ld, (const T*) gate, gate_ld, (const T*) t, t_ld, (const T*) w2, w0, u, norm_w, tok_pos, slots, heads, dim, vdim, rank, eps, w_vec)
     MIX_DISPATCH_T(dtype, if (by4) TS_LAUNCH(4); else TS_LAUNCH(1));
     #undef TS_LAUNCH
     return mix_check_launch("mix_timemix_step");

@@ -1002,10 +1002,11 @@ TIMEMIX_FUSED_VDIM = 64       # head norm and gate run in the prompt kernel up t
 
 
 def token_shift(out, h_view, last, mu, sb):
-    """out [mixes, n, width] = h + (h' - h) mu[m], h' the previous token's row (the step's own, or last [slots, width], or zeros); a sequence's last row goes into `last`."""
+    """out [mixes, n, width] = h + (h' - h) mu[m], h' the previous token's row (the step's own, or from last [slots, width], or zeros); a sequence's
+    last row goes into `last`."""
     mixes, n, width = out.shape
     _f32c(mu, "mu")
-    _req(out.is_contiguous() and mu.shape == (mixes, width) and h_view.shape[0] == n and last.is_contiguous() and last.dim() == 2 and last.shape[1] == width
+    _req(out.is_contiguous() and mu.shape == (mixes, width) and h_view.shape[0] == n and last.is_contiguous() and last.shape[1:] == (width,)
          and out.dtype == h_view.dtype == last.dtype, "token_shift: shapes")
     for t, nm in ((sb.tok_seq, "tok_seq"), (sb.tok_pos, "tok_pos"), (sb.slots, "slots"), (sb.pos0, "pos0"), (sb.len_after, "len_after")):
         _i32c(t, nm)
@@ -1014,25 +1015,25 @@ def token_shift(out, h_view, last, mu, sb):
                                                _p(sb.len_after), n, width, code(out.dtype), _stream(out)))
 
 
-def decay_log(out, t_view, w2, w0):
-    """out [n, channels] float32 = -exp(w0 + w2 tanh(t)): the logarithms of the decays."""
+def decay_log2(out, t_view, w2, w0):
+    """out [n, channels] float32 = -log2(e) exp(w0 + w2 tanh(t)): base-2 logarithms of the decays."""
     n, channels = out.shape
     _f32c(out, "out"); _f32c(w0, "w0")
-    _req(w2.is_contiguous() and w2.shape[0] == channels == w0.numel() and t_view.shape[0] == n and w2.dtype == t_view.dtype, "decay_log: shapes")
-    _check(_lib.mixlib().exl3_mix_decay_log(_p(out), _p(t_view), _view(t_view, w2.shape[1], "t"), _p(w2), _p(w0), n, channels, w2.shape[1], code(w2.dtype), _stream(out)))
+    _req(w2.is_contiguous() and w2.shape[0] == channels == w0.numel() and t_view.shape[0] == n and w2.dtype == t_view.dtype, "decay_log2: shapes")
+    _check(_lib.mixlib().exl3_mix_decay_log2(_p(out), _p(t_view), _view(t_view, w2.shape[1], "t"), _p(w2), _p(w0), n, channels, w2.shape[1], code(w2.dtype), _stream(out)))
 
 
-def timemix(o, out, gate_view, norm_w, eps: float, state, r_view, k_view, v_view, logw, u, cu, slots, pos0, segments: tuple[int, int] | None = None):
-    """Prompt steps.  state [slots, heads, dim, vdim] float32, logw [n, heads * dim] float32, u [heads * dim] float32.  Either o [n, heads, vdim] float32 receives the
+def timemix(o, out, gate_view, norm_w, eps: float, state, r_view, k_view, v_view, log2w, u, cu, slots, pos0, segments: tuple[int, int] | None = None):
+    """Prompt steps.  state [slots, heads, dim, vdim] float32, log2w [n, heads * dim] float32, u [heads * dim] float32.  Either o [n, heads, vdim] float32 receives the
     read-outs, or (vdim <= TIMEMIX_FUSED_VDIM) out [n, heads * vdim] the heads after norm, norm_w and silu gate.  segments = (segs, seg_len): every sequence cut into parallel
     segments; None: one chain of tiles per sequence."""
     n = r_view.shape[0]
     heads, dim, vdim = state.shape[1:]
-    _f32c(state, "state"); _f32c(logw, "logw"); _f32c(u, "u")
+    _f32c(state, "state"); _f32c(log2w, "log2w"); _f32c(u, "u")
     for t, nm in ((cu, "cu"), (slots, "slots"), (pos0, "pos0")):
         _i32c(t, nm)
     batch = slots.numel()
-    _req(logw.shape == (n, heads * dim) and u.numel() == heads * dim and cu.numel() == batch + 1 and pos0.numel() == batch and k_view.shape[0] == n and v_view.shape[0] == n
+    _req(log2w.shape == (n, heads * dim) and u.numel() == heads * dim and cu.numel() == batch + 1 and pos0.numel() == batch and k_view.shape[0] == n and v_view.shape[0] == n
          and r_view.dtype == k_view.dtype == v_view.dtype, "timemix: shapes")
     _req((o is None) != (out is None), "timemix: either the read-outs or the gated heads")
     oa = (None, 0, None, 0, None)
@@ -1046,7 +1047,7 @@ def timemix(o, out, gate_view, norm_w, eps: float, state, r_view, k_view, v_view
     seg_state = torch.empty((batch * segs, heads, dim, vdim), dtype=torch.float32, device=state.device) if segs > 1 else None
     seg_decay = torch.empty((batch * segs, heads, dim), dtype=torch.float32, device=state.device) if segs > 1 else None
     _check(_lib.mixlib().exl3_mix_timemix(_p(o), *oa, eps, _p(state), _p(r_view), _view(r_view, heads * dim, "r"), _p(k_view), _view(k_view, heads * dim, "k"), _p(v_view),
-                                           _view(v_view, heads * vdim, "v"), _p(logw), _p(u), _p(cu), _p(slots), _p(pos0), batch, heads, dim, vdim, segs, seg_len, _p(seg_state),
+                                           _view(v_view, heads * vdim, "v"), _p(log2w), _p(u), _p(cu), _p(slots), _p(pos0), batch, heads, dim, vdim, segs, seg_len, _p(seg_state),
                                            _p(seg_decay), code(r_view.dtype), _stream(state)))
 
 
@@ -1061,3 +1062,34 @@ def timemix_step(out, state, r_view, k_view, v_view, gate_view, t_view, w2, w0, 
                                                 _p(v_view), _view(v_view, heads * vdim, "v"), _p(gate_view), _view(gate_view, heads * vdim, "gate"), _p(t_view),
                                                 _view(t_view, w2.shape[1], "t"), _p(w2), _p(w0), _p(u), _p(norm_w), _p(tok_pos), _p(slots), n, heads, dim, vdim, w2.shape[1], eps,
                                                 code(out.dtype), _stream(out)))
+
+
+# ---- matrix products of few rows (csrc/mix_skinny.hip) --------------------------------------------------------------------------------------------------
+SKINNY_MAX_ROWS = 16
+
+
+def skinny_ok(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """x [..., n, K] against w [.., K]: few rows, bfloat16, 16-byte aligned rows."""
+    return (x.dtype == w.dtype == torch.bfloat16 and 0 < x.shape[-2] <= SKINNY_MAX_ROWS and x.shape[-1] % 8 == 0 and x.stride(-1) == 1 == w.stride(-1) and x.stride(-2) % 8 == 0
+            and w.stride(-2) % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and x.is_cuda)
+
+
+def skinny(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None) -> torch.Tensor:
+    """x [n, K] W^T + bias for few rows: the weights w [rows, K] (any row stride) are streamed once."""
+    n, K = x.shape
+    rows = w.shape[0]
+    _req(skinny_ok(x, w) and w.shape[1] == K and (bias is None or (bias.numel() == rows and bias.is_contiguous() and bias.dtype == x.dtype)), "skinny: shapes")
+    out = torch.empty((n, rows), dtype=x.dtype, device=x.device)
+    _check(_lib.mixlib().exl3_mix_skinny(_p(out), rows, 0, None, 0, _p(x), max(x.stride(0), K), 0, _p(w), max(w.stride(0), K), _p(bias), n, K, 1, rows, 0, _stream(x)))
+    return out
+
+
+def skinny_stack(x: torch.Tensor, w: torch.Tensor, rows: int) -> tuple[torch.Tensor, torch.Tensor]:
+    """x [mats + 1, n, K], w [mats * rows + tail, K] contiguous: every matrix with its own x in one launch; returns [mats, n, rows] and [n, tail]."""
+    m1, n, K = x.shape
+    mats = m1 - 1
+    tail = w.shape[0] - mats * rows
+    _req(skinny_ok(x, w) and x.is_contiguous() and w.is_contiguous() and w.shape[1] == K and tail > 0 and mats > 0, "skinny_stack: shapes")
+    out, last = torch.empty((mats, n, rows), dtype=x.dtype, device=x.device), torch.empty((n, tail), dtype=x.dtype, device=x.device)
+    _check(_lib.mixlib().exl3_mix_skinny(_p(out), rows, n * rows, _p(last), tail, _p(x), K, n * K, _p(w), K, None, n, K, mats, rows, tail, _stream(x)))
+    return out, last

@@ -69,6 +69,13 @@ def _f32(stc, key: str, device) -> torch.Tensor:
     return stc.get_tensor(key, device="cpu").to(torch.float32).to(device).contiguous()
 
 
+def linear(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None) -> torch.Tensor:
+    """x W^T + bias: steps of few rows stream the weights through the library's own kernel, everything else is a vendor product."""
+    if mix_ops.skinny_ok(x, w):
+        return mix_ops.skinny(x, w, bias)
+    return F.linear(x, w, bias)
+
+
 class FusedInput:
     """Linears that read the same input, stacked into one weight: one matrix product instead of several, and every consumer kernel takes its
     column block in place (row stride = total width).  Parts without a bias get zeros in the fused bias (adding zero is exact)."""
@@ -87,7 +94,7 @@ class FusedInput:
             self.offsets[n] = (at, s); at += s
 
     def __call__(self, h: torch.Tensor) -> dict[str, torch.Tensor]:
-        out = F.linear(h, self.weight, self.bias)
+        out = linear(h, self.weight, self.bias)
         p = {n: out[:, a: a + s] for n, (a, s) in self.offsets.items()}
         p[self.ALL] = out                     # the whole product, for a consumer that reads several neighbouring parts as one block
         return p
@@ -137,7 +144,7 @@ class SlidingSinkAttention:
         else:
             mix_ops.attn_prefill(out, p["q"], p["k"], v_norm, p.get("g"), self.sink, sb.cu, sb.tok_seq, sb.tok_pos, self.heads, self.scale, self.window,
                                  max_rows=sb.max_rows)
-        return F.linear(out, self.w_o), p
+        return linear(out, self.w_o), p
 
 
 class GatedLinearAttention:
@@ -182,7 +189,7 @@ class GatedLinearAttention:
                          segments=self.segments(sb))
         out = torch.empty((sb.n, self.heads * self.vdim), dtype=self.dtype, device=h.device)
         mix_ops.gla_out(out, o, self.norm_w, p["g"], self.eps)
-        return F.linear(out, self.w_o), p
+        return linear(out, self.w_o), p
 
 
 class PolyNormMLP:
@@ -200,7 +207,7 @@ class PolyNormMLP:
         p = self.inp(h)
         a = torch.empty((sb.n, self.ff), dtype=self.dtype, device=h.device)
         mix_ops.polynorm(a, p["up"], self.coef, self.eps)
-        return F.linear(a, self.w_down), p
+        return linear(a, self.w_down), p
 
 
 def rotary_frequencies(dims: int, base: float, scaling: dict | None = None) -> tuple[torch.Tensor, float]:
@@ -322,8 +329,8 @@ class LatentAttention:
         else:
             out = torch.empty((sb.n, H * dv), dtype=self.dtype, device=h.device)
             c = ckr[:, :rank]
-            k = F.linear(c, self.w_uk_padded)                                    # [n, H * (d + r)], the rotated slots still zero
-            v = F.linear(c, self.w_uv).view(sb.n, H, dv)
+            k = linear(c, self.w_uk_padded)                                    # [n, H * (d + r)], the rotated slots still zero
+            v = linear(c, self.w_uv).view(sb.n, H, dv)
             mix_ops.latent_fill_k(k, ckr, H, d, r, rank)
             if self.has_gate:
                 o = torch.empty((sb.n, H * dv), dtype=self.dtype, device=h.device)
@@ -331,7 +338,7 @@ class LatentAttention:
                 mix_ops.heads_gate(out, o, H * dv, dv, p["g"], H, dv)
             else:
                 mix_ops.attn_prefill(out, q, k, v, None, self.sink, sb.cu, sb.tok_seq, sb.tok_pos, H, self.scale, self.window, max_rows=sb.max_rows)
-        return F.linear(out, self.w_o), p
+        return linear(out, self.w_o), p
 
 
 class PagedLatentAttention(LatentAttention):
@@ -381,7 +388,7 @@ class PagedLatentAttention(LatentAttention):
             if not sb.decode:
                 sb.shared["latent", self.layer] = ckr
         mix_ops.latent_rows(sb.tok_seq, sb.tok_pos, sb.slots, self.eps, self.freq, self.rot_mag, self.interleaved, dkv=dkv, dq=(cq, p["dq"], self.q_norm))
-        q = F.linear(cq, self.w_uq)
+        q = linear(cq, self.w_uq)
         if self.rot_dims:
             mix_ops.rotate_heads(q, sb.tok_pos, self.freq, self.rot_mag, self.interleaved, H, self.qk, d)
         if sb.decode:
@@ -394,8 +401,8 @@ class PagedLatentAttention(LatentAttention):
             return
         ckr = sb.shared["latent", self.layer if self.kv_from is None else self.kv_from]
         c = ckr[:, :rank]
-        k = F.linear(c, self.w_uk_padded)                                        # [n, H * (d + r)], the rotated slots still zero
-        v = F.linear(c, self.w_uv)
+        k = linear(c, self.w_uk_padded)                                        # [n, H * (d + r)], the rotated slots still zero
+        v = linear(c, self.w_uv)
         mix_ops.latent_fill_k(k, ckr, H, d, r, rank)
         mix_ops.attn_prefill_maps(out, q, k, v, p.get("g"), self.sink, sb.cu, sb.tok_seq, sb.tok_pos, H, H, 1, self.qk, dv, self.scale, 0.0, self.EVERY, mix_ops.MASK_WINDOW,
                                   max_rows=sb.max_rows)
@@ -403,7 +410,7 @@ class PagedLatentAttention(LatentAttention):
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
         self.attend(h, sb, state, out)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class KeptWindowAttention:
@@ -483,7 +490,7 @@ class KeptWindowAttention:
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
         self.attend(h, sb, state, out)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class Retention:
@@ -540,7 +547,7 @@ class Retention:
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
         self.attend(h, sb, state, out)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class TimeMix:
@@ -550,7 +557,7 @@ class TimeMix:
     on the result (folded into the float32 weight)."""
     # prompt steps whose longest sequence has at least this many rows are cut into parallel segments, enough of them for about this many workgroups
     SEGMENT_MIN_ROWS = 256
-    SEGMENT_TARGET_WORKGROUPS = 1024
+    SEGMENT_TARGET_WORKGROUPS = 768          # three fit a CU
     SEGMENT_ROWS = 64                        # a segment's shortest length
 
     def __init__(self, width: int, heads: int, dim: int, eps: float, out_scale: float = 1.0):
@@ -563,14 +570,17 @@ class TimeMix:
     def load(self, stc, prefix: str, dtype, device, extra_parts=()):
         self.inp = FusedInput(list(extra_parts)) if extra_parts else None
         n = self.heads * self.dim
-        # r, k, v, g as one batched product over their mixes: [4, width, heads * dim]
-        self.w_rkvg = torch.stack([_w(stc, prefix + nm, dtype, device).t() for nm in ("r", "k", "v", "g")]).contiguous()
+        parts = [_w(stc, prefix + nm, dtype, device) for nm in ("r", "k", "v", "g", "w1")]
+        assert all(t.shape == (n, self.width) for t in parts[:4]) and parts[4].shape[1] == self.width
+        self.rank = parts[4].shape[0]
+        self.w_in = torch.cat(parts, dim=0).contiguous()                                 # one behind the other: a step of few rows streams them in one launch
+        self.w_mix = list(self.w_in.split([n] * 4 + [self.rank]))                        # views
         self.mu = torch.stack([_f32(stc, prefix + "mu." + nm, device) for nm in ("r", "k", "v", "g", "w")]).contiguous()
-        self.w1, self.w2 = _w(stc, prefix + "w1", dtype, device), _w(stc, prefix + "w2", dtype, device)
+        self.w2 = _w(stc, prefix + "w2", dtype, device)
         self.w0, self.u = _f32(stc, prefix + "w0", device), _f32(stc, prefix + "u", device).reshape(-1).contiguous()
         self.norm_w = (_f32(stc, prefix + "norm", device) * self.out_scale).contiguous()
         self.w_o = _w(stc, prefix + "o", dtype, device)
-        assert self.w_rkvg.shape == (4, self.width, n) and self.mu.shape == (5, self.width) and self.w1.shape == (self.w2.shape[1], self.width) and self.w2.shape[0] == n
+        assert self.mu.shape == (5, self.width) and self.w2.shape == (n, self.rank)
         assert self.w0.numel() == self.u.numel() == self.norm_w.numel() == n and self.w_o.shape == (self.width, n)
         self.dtype = dtype
 
@@ -591,23 +601,26 @@ class TimeMix:
     def attend(self, h: torch.Tensor, sb: StepBatch, state: dict, out: torch.Tensor):
         mix = torch.empty((5, sb.n, self.width), dtype=self.dtype, device=h.device)
         mix_ops.token_shift(mix, h, state["last"], self.mu, sb)
-        r, k, v, g = torch.bmm(mix[:4], self.w_rkvg).unbind(0)
-        t = F.linear(mix[4], self.w1)
+        if mix_ops.skinny_ok(mix, self.w_in):
+            y, t = mix_ops.skinny_stack(mix, self.w_in, self.out_width)
+            r, k, v, g = y.unbind(0)
+        else:
+            r, k, v, g, t = (linear(x, w) for x, w in zip(mix.unbind(0), self.w_mix))
         if sb.decode:
             mix_ops.timemix_step(out, state["S"], r, k, v, g, t, self.w2, self.w0, self.u, self.norm_w, sb.tok_pos, sb.slots, self.eps)
             return
-        logw = torch.empty((sb.n, self.out_width), dtype=torch.float32, device=h.device)
-        mix_ops.decay_log(logw, t, self.w2, self.w0)
+        log2w = torch.empty((sb.n, self.out_width), dtype=torch.float32, device=h.device)
+        mix_ops.decay_log2(log2w, t, self.w2, self.w0)
         fused = self.dim <= mix_ops.TIMEMIX_FUSED_VDIM
         o = None if fused else torch.empty((sb.n, self.heads, self.dim), dtype=torch.float32, device=h.device)
-        mix_ops.timemix(o, out if fused else None, g, self.norm_w, self.eps, state["S"], r, k, v, logw, self.u, sb.cu, sb.slots, sb.pos0, segments=self.segments(sb))
+        mix_ops.timemix(o, out if fused else None, g, self.norm_w, self.eps, state["S"], r, k, v, log2w, self.u, sb.cu, sb.slots, sb.pos0, segments=self.segments(sb))
         if not fused:
             mix_ops.head_norm_gate(out, o, self.norm_w, g, mix_ops.GATE_SILU, self.eps)
 
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
         self.attend(h, sb, state, out)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class SummedMixers:
@@ -640,7 +653,7 @@ class SummedMixers:
     def forward(self, h: torch.Tensor, sb: StepBatch, state: dict) -> torch.Tensor:
         out = torch.empty((sb.n, self.out_width), dtype=self.dtype, device=h.device)
         self.attend(h, sb, state, out)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class ActMLP:
@@ -659,7 +672,7 @@ class ActMLP:
         p = self.inp(h)
         a = torch.empty((sb.n, self.ff), dtype=self.dtype, device=h.device)
         mix_ops.act(a, p["up"], self.kind)
-        return F.linear(a, self.w_down), p
+        return linear(a, self.w_down), p
 
 
 class GatedMLP:
@@ -692,7 +705,7 @@ class GatedMLP:
         a, p = self.hidden(h)
         if add_to is not None:
             return torch.addmm(add_to, a, self.w_down.t()), p
-        return F.linear(a, self.w_down), p
+        return linear(a, self.w_down), p
 
 
 class TokenSide:
@@ -710,10 +723,10 @@ class TokenSide:
         self.dtype = dtype
 
     def forward(self, xc: torch.Tensor, sb: StepBatch) -> torch.Tensor:
-        gate = F.linear(xc, self.w_gate)
+        gate = linear(xc, self.w_gate)
         g = torch.empty((sb.n, self.dim), dtype=self.dtype, device=xc.device)
         mix_ops.token_gate(g, gate, self.table, self.index * self.dim, sb.tokens)
-        return F.linear(g, self.w_proj)
+        return linear(g, self.w_proj)
 
 
 class PreNormBlock:
@@ -955,7 +968,7 @@ class DifferentialAttention:
             # matrix cores: both maps of a head in one workgroup, combined in the epilogue
             mix_ops.attn_prefill_diff(out, p["q"], p["k"], p["v"], p.get("g"), sb.cu, H, G, d, dv, self.scale, self.softcap, self.span, self.mask, self.lam, self.diff,
                                       self.eps, sb.max_rows)
-            return F.linear(out, self.w_o, self.b_o), p
+            return linear(out, self.w_o, self.b_o), p
         a = torch.empty((sb.n, H * M * dv), dtype=torch.float32, device=h.device)      # the maps' weighted sums stay float32 until they are combined
         if sb.decode:
             mix_ops.attn_decode_maps(a, p["q"], state["ring_k"], state["ring_v"], None, None, sb.slots, sb.len_after, H, M, self.scale, self.softcap, self.mask)
@@ -963,7 +976,7 @@ class DifferentialAttention:
             mix_ops.attn_prefill_maps(a, p["q"], p["k"], p["v"], None, None, sb.cu, sb.tok_seq, sb.tok_pos, H, G, M, d, dv, self.scale, self.softcap, self.span,
                                       self.mask, max_rows=sb.max_rows)
         mix_ops.diff_combine(out, a, self.lam, self.diff, self.eps, p.get("g"), H, dv)
-        return F.linear(out, self.w_o, self.b_o), p
+        return linear(out, self.w_o, self.b_o), p
 
 
 class CanonBlock:
@@ -1078,7 +1091,7 @@ class SigmoidAttention(_SideMixer):
             mix_ops.sigattn_decode(out, q, kp, vp, self.bias, table, sb.slots, sb.len_after, H, G, d, dv, self.scale)
         else:
             mix_ops.sigattn_prefill(out, q, k, v, self.bias, sb.cu, sb.tok_seq, H, G, d, dv, self.scale, sb.max_rows)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class MatrixLSTM(_SideMixer):
@@ -1114,7 +1127,7 @@ class MatrixLSTM(_SideMixer):
                            sb.cu, sb.slots, sb.pos0, self.q_scale, self.cap)
         out = torch.empty((sb.n, H * dv), dtype=self.dtype, device=o.device)
         mix_ops.head_norm_gate(out, o, self.norm_w, p[t + "g"], mix_ops.GATE_SIGMOID, self.eps)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class GatedDeltaRule(_SideMixer):
@@ -1164,7 +1177,7 @@ class GatedDeltaRule(_SideMixer):
         mix_ops.delta_scan(o, state[t + "S"], q, k, v, beta, decay, sb.cu, sb.slots, sb.pos0, G)
         out = torch.empty((sb.n, H * dv), dtype=self.dtype, device=dev)
         mix_ops.head_norm_gate(out, o, self.norm_w, p[t + "g"], mix_ops.GATE_SILU, self.eps)
-        return F.linear(out, self.w_o)
+        return linear(out, self.w_o)
 
 
 class ParallelMixer(_SideMixer):
@@ -1263,7 +1276,7 @@ class DualNormBlock:
         self.mixer.attend(h1, sb, state, cat[:, : self.split])
         if self.mlp is not None:
             self.mlp.hidden(h2, out=cat[:, self.split:])
-        return F.linear(cat, self.w_out)
+        return linear(cat, self.w_out)
 
 
 class PostNormBlock:

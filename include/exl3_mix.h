@@ -385,22 +385,27 @@ int exl3_mix_retention_step(void* out, int64_t out_ld, float* state, const void*
                             const void* gate, int64_t gate_ld, const float* pw, int pw_ld, const float* freq, int rot_dims, int interleaved, const int32_t* tok_pos,
                             const int32_t* slots, int n, int heads, int dim, int vdim, float k_scale, float eps, int dtype, void* stream);
 
+/* Matrix products of few rows, bfloat16 (mix_skinny.hip): for m < mats  out[m][i] = x[m][i] W_m^T + bias_m (rows outputs; bias [mats rows + tail] or NULL), and with tail > 0 one
+ * more product of `tail` outputs, out_tail[i] = x[mats][i] W^T.  w: the matrices one behind the other, [mats rows + tail][K] with row stride w_ld.  K a multiple of 8, rows of x and
+ * w 16-byte aligned; weights are read once per sixteen rows of x. */
+int exl3_mix_skinny(void* out, int64_t out_ld, int64_t out_mat, void* out_tail, int64_t tail_ld, const void* x, int64_t x_ld, int64_t x_mat, const void* w, int64_t w_ld,
+                    const void* bias, int n, int K, int mats, int rows, int tail, void* stream);
+
 /* ---- time mixing with a decay per key channel and token and a bonus for the current token (mix_timemix.hip) ---- */
 
-/* out[m][n] = h[n] + (h'[n] - h[n]) mu[m], m < mixes; h'[n]: the row before n in its sequence -- the step's own, or `last` [slots][width], or zeros ahead of the
- * first token.  A sequence's last row goes into `last`.  out [mixes][n][width], mu [mixes][width]. */
+/* out[m][n] = h[n] + (h'[n] - h[n]) mu[m], m < mixes; h'[n]: the row before n in its sequence -- the step's own, or from `last` [slots][width], or zeros ahead of the first token.  A sequence's last row goes into `last`.  out [mixes][n][width], mu [mixes][width]. */
 int exl3_mix_token_shift(void* out, const void* h, int64_t h_ld, void* last, const float* mu, int mixes, const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots,
                          const int32_t* pos0, const int32_t* len_after, int n, int width, int dtype, void* stream);
-/* Logarithms of the decays: out[n][c] = -exp(w0[c] + sum_r tanh(t[n][r]) w2[c][r]), c < channels (float32 throughout). */
-int exl3_mix_decay_log(float* out, const void* t, int64_t t_ld, const void* w2, const float* w0, int n, int channels, int rank, int dtype, void* stream);
-/* Per head o_t = (S + diag(u) k_t v_t^T)^T r_t, then S <- diag(w_t) S + k_t v_t^T with w = exp(logw) [n][heads * dim], u [heads * dim].  o [n][heads][vdim] float32, or
+/* Base-2 logarithms of the decays: out[n][c] = -log2(e) exp(w0[c] + sum_r tanh(t[n][r]) w2[c][r]), c < channels (float32 throughout). */
+int exl3_mix_decay_log2(float* out, const void* t, int64_t t_ld, const void* w2, const float* w0, int n, int channels, int rank, int dtype, void* stream);
+/* Per head o_t = (S + diag(u) k_t v_t^T)^T r_t, then S <- diag(w_t) S + k_t v_t^T with w = 2^log2w [n][heads * dim], u [heads * dim].  o [n][heads][vdim] float32, or
  * with `out` (vdim <= 64) the heads after norm and gate, o / sqrt(mean(o^2) + eps) * norm_w[heads * vdim] * silu(gate).  state [slots][heads][dim][vdim] float32;
  * dim <= 256, vdim <= 1024.  segs > 1: every sequence in `segs` segments of seg_len rows that run in parallel; seg_state holds batch * segs * heads * dim * vdim floats,
  * seg_decay batch * segs * heads * dim. */
 int exl3_mix_timemix(float* o, void* out, int64_t out_ld, const void* gate, int64_t gate_ld, const float* norm_w, float eps, float* state, const void* r, int64_t r_ld,
-                     const void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* logw, const float* u, const int32_t* cu, const int32_t* slots,
+                     const void* k, int64_t k_ld, const void* v, int64_t v_ld, const float* log2w, const float* u, const int32_t* cu, const int32_t* slots,
                      const int32_t* pos0, int batch, int heads, int dim, int vdim, int segs, int seg_len, float* seg_state, float* seg_decay, int dtype, void* stream);
-/* One row per sequence: decays (as exl3_mix_decay_log), read-out, state update, head norm and gate. */
+/* One row per sequence: decays exp(-exp(w0 + w2 tanh(t))), read-out, state update, head norm and gate. */
 int exl3_mix_timemix_step(void* out, int64_t out_ld, float* state, const void* r, int64_t r_ld, const void* k, int64_t k_ld, const void* v, int64_t v_ld, const void* gate,
                           int64_t gate_ld, const void* t, int64_t t_ld, const void* w2, const float* w0, const float* u, const float* norm_w, const int32_t* tok_pos,
                           const int32_t* slots, int n, int heads, int dim, int vdim, int rank, float eps, int dtype, void* stream);
