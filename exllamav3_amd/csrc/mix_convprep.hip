@@ -1,5 +1,5 @@
-// What attention reads when its projections pass a short causal convolution over time first: per channel of q | k | v  y_t = sum_j w[j] u_(t - taps + 1 + j) (zeros
-// before the sequence's start), then per query / key head the RMS norm and the rotation of qk_prep (mix_diffattn.hip), and the rows that the sequence keeps go
+// What attention reads when its projected rows are filtered along the tokens first: every channel of q | k | v becomes the weighted sum of its last `taps` values,
+// sum_i w[taps - 1 - i] x_(t - i) (nothing ahead of the first token), then per query / key head the RMS norm and the rotation of qk_prep (mix_diffattn.hip), and the rows that the sequence keeps go
 // into its rings of keys and values.  One launch for prompt steps and for steps of one row per sequence: a row's predecessors are the step's own rows where the
 // sequence has them in the step and the slot's ring of the last taps - 1 projected rows otherwise.  Sums, norms, angles are float32; the result is rounded once.
 //

@@ -1,5 +1,5 @@
 // Time mixing with a decay per key channel and token and a bonus for the current token (RWKV-style).  Per head, with decays w_t in (0, 1] given by their base-2 logarithms:
-//   o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,   S_t = diag(w_t) S_(t-1) + k_t v_t^T
+//   o = S^T r + (sum_c r_c u_c k_c) v,   then for every key channel c   S[c] <- w_c S[c] + k_c v
 // Everything that enters the recurrence besides the projections is float32; the state [slot][head][dim][vdim] is float32.
 //
 //   token_shift    what the projections read: h + (h' - h) mu_m for every mix m, h' the previous token's row (of the step, or from the slot)

@@ -1,6 +1,6 @@
 """
-Menerax: a decoder-only model of post-norm blocks over a float32 stream: x <- x + norm1(mixer(x)), then x <- x + norm2(ff(x)), the norms on the sublayers' outputs and
-the sublayers reading x itself.  A layer's mixer is latent attention over every earlier token (a cached low-rank latent and one rotated key part per token, queries
+Menerax: a decoder-only model of post-norm blocks over a float32 stream: x += norm1(mixer(x)); x += norm2(ff(x)), with the norms behind the sublayers and no norm
+ahead of them.  A layer's mixer is latent attention over every earlier token (a cached low-rank latent and one rotated key part per token, queries
 through a latent of their own, one output gate per head), or two mixers side by side, scaled and added: sliding-window attention that keeps the first tokens of a
 sequence visible (biases, short convolutions on q / k / v, normed queries and keys, soft-capped scores, element-wise output gate) and RWKV-style time mixing.  The
 feed-forward is a gated layer with a clamped swish, or none.  A layer may use an earlier one's weights with a cache of its own.  The order of layers and every size and

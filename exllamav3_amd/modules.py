@@ -2,7 +2,8 @@
 Building blocks of the unquantized mixer models: each mechanism is one class with its constants as constructor arguments, its tensors
 read through the framework's SafetensorsCollection, its per-slot state declared as StateSpec, and a forward over a packed StepBatch that
 runs the kernels of libexl3_mix.so (mix_ops) around vendor matrix products (torch.nn.functional.linear: hipBLASLt / rocBLAS with
-float32 accumulation; true float32 when the model runs in float32).
+float32 accumulation; true float32 when the model runs in float32).  Products of up to 16 bfloat16 rows go to the library's weight-streaming
+kernel instead (linear).
 
     FusedInput              several linears over one input as one matrix product, outputs as column views
     SlidingSinkAttention    grouped-query attention over a sliding window, optional learned sink in the softmax denominator, optional unit-RMS
@@ -46,7 +47,7 @@ float32 accumulation; true float32 when the model runs in float32).
     TimeMix                 RWKV-style time mixing: token shift, a decay per key channel and token from a low-rank product, a bonus for the current token, float32 state,
                             per-head unit RMS, silu gate
     SummedMixers            two mixers side by side, scaled and added inside ONE output product
-    PostNormBlock           x += norm1(mixer(x)); x += norm2(ff(x)): the norms sit on the sublayers' outputs, which read the stream itself
+    PostNormBlock           x += norm1(mixer(x)); x += norm2(ff(x)): the norms sit behind the sublayers, whose input is the unnormed stream
     DualNormBlock           x += mixer(norm1(x)) + ff(norm2(x)): both norms from one pass over the stream, both output projections as ONE product over
                             [mixer's heads | hidden activation]
 
@@ -417,8 +418,8 @@ class KeptWindowAttention:
     """H query heads over G key/value heads.  A row sees the last `size` positions up to itself and the sequence's first `keep_first` positions, which keep
     their true positions.  Rotary positions on the first rot_dims entries of queries and keys; tied: the values are the keys before their rotation (no W_v).
     Optional sink (one more term of the denominator per head) and output gate per value element.  A slot holds keep_first + size rows of keys and values: the
-    first positions' for good, and a ring of the last `size` of the others.  Optional: biases of the q / k / v projections; a short causal convolution over time on every
-    channel of q, k and v (taps > 0; the slot also holds the last taps - 1 projected rows); an RMS norm of every query / key head with a plain weight over dim; scores
+    first positions' for good, and a ring of the last `size` of the others.  Optional: biases of the q / k / v projections; a filter of `taps` tokens along
+    every channel of the projected rows (taps > 0; the slot also holds the last taps - 1 of them); an RMS norm of every query / key head with a plain weight over dim; scores
     soft-capped to softcap tanh(score / softcap); a factor on the result (out_scale)."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, size: int, keep_first: int, rot_dims: int, rot_base: float,
@@ -551,9 +552,9 @@ class Retention:
 
 
 class TimeMix:
-    """RWKV-style time mixing.  With h' the previous token's h (zeros ahead of the first), each of r, k, v, g, w reads its own mix h + (h' - h) mu; r, k, v per head, gate =
-    silu(W_g mix_g); decay w = exp(-exp(w0 + W_w2 tanh(W_w1 mix_w))) per head and key channel.  o_t = (S + diag(u) k v^T)^T r, then S <- diag(w) S + k v^T; each head's o over
-    its root mean square, times a weight over all heads' values, times the gate.  Per slot: S [heads, dim, dim] float32 and the last token's h.  out_scale: a factor
+    """RWKV-style time mixing.  Five inputs x_m = h + mu_m (h_prev - h), h_prev the row of the token before (zero ahead of the first), one each for r, k, v, the gate silu(W_g x_g)
+    and the decay: log w = -exp(w0 + W_2 tanh(W_1 x_w)) per head and key channel c.  o = S^T r + (sum_c r_c u_c k_c) v, then S[c] <- w_c S[c] + k_c v; every head of o is
+    scaled to unit RMS, then weighted over all heads' values and gated.  Per slot: S [heads, dim, dim] float32 and the last token's h.  out_scale: a factor
     on the result (folded into the float32 weight)."""
     # prompt steps whose longest sequence has at least this many rows are cut into parallel segments, enough of them for about this many workgroups
     SEGMENT_MIN_ROWS = 256
@@ -1280,8 +1281,8 @@ class DualNormBlock:
 
 
 class PostNormBlock:
-    """x <- x + norm1(mixer(x)), then x <- x + norm2(ff(x)) (if a feed-forward): RMS norms on the sublayers' outputs, whose stored weights are deviations from one; the
-    sublayers read the float32 stream itself, in the activation type.  Every update of the stream is one kernel: the norm of the sublayer's output, the addition and
+    """x += norm1(mixer(x)) and, with a feed-forward, x += norm2(ff(x)): RMS norms behind the sublayers, with weights stored as deviations from one; mixer and feed-forward
+    are given the float32 stream unnormed, in the activation type.  Every update of the stream is one kernel: the norm of the sublayer's output, the addition and
     the copy of the stream that the next sublayer reads."""
 
     def __init__(self, width: int, eps: float, mixer, mlp):

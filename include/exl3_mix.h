@@ -257,7 +257,7 @@ int exl3_mix_qk_prep(void* q, int64_t q_ld, const void* k, int64_t k_ld, void* k
                      const int32_t* tok_seq, const int32_t* tok_pos, const int32_t* slots, const int32_t* len_after,
                      int n, int q_heads, int k_heads, int v_heads, int dim, int vdim, int window, int keep_first, int dtype, void* stream);
 
-/* The same for queries, keys and values whose projections pass a short causal convolution over time (mix_convprep.hip).  x [n][q_heads dim | kv_heads dim |
+/* The same for queries, keys and values whose projected rows are filtered along the tokens, channel by channel (mix_convprep.hip).  x [n][q_heads dim | kv_heads dim |
  * kv_heads vdim] (row stride x_ld); conv_w [taps][C] over those C columns, the last tap is the row's own; predecessors come from the step's own rows or from
  * conv_ring [slots][taps - 1][C], which keeps the last taps - 1 projected rows of a sequence; zeros before its start.  out [n][C]: normed and rotated
  * queries and keys, convolved values.  ring_k [slots][rows][kv_heads][dim], ring_v [slots][rows][kv_heads][vdim] as above (keep_first).  1..16 taps. */
@@ -398,7 +398,7 @@ int exl3_mix_token_shift(void* out, const void* h, int64_t h_ld, void* last, con
                          const int32_t* pos0, const int32_t* len_after, int n, int width, int dtype, void* stream);
 /* Base-2 logarithms of the decays: out[n][c] = -log2(e) exp(w0[c] + sum_r tanh(t[n][r]) w2[c][r]), c < channels (float32 throughout). */
 int exl3_mix_decay_log2(float* out, const void* t, int64_t t_ld, const void* w2, const float* w0, int n, int channels, int rank, int dtype, void* stream);
-/* Per head o_t = (S + diag(u) k_t v_t^T)^T r_t, then S <- diag(w_t) S + k_t v_t^T with w = 2^log2w [n][heads * dim], u [heads * dim].  o [n][heads][vdim] float32, or
+/* Per head o = S^T r + (sum_c r_c u_c k_c) v, then S[c] <- w_c S[c] + k_c v for every key channel c, with w = 2^log2w [n][heads * dim], u [heads * dim].  o [n][heads][vdim] float32, or
  * with `out` (vdim <= 64) the heads after norm and gate, o / sqrt(mean(o^2) + eps) * norm_w[heads * vdim] * silu(gate).  state [slots][heads][dim][vdim] float32;
  * dim <= 256, vdim <= 1024.  segs > 1: every sequence in `segs` segments of seg_len rows that run in parallel; seg_state holds batch * segs * heads * dim * vdim floats,
  * seg_decay batch * segs * heads * dim. */

@@ -81,7 +81,7 @@ def kept_window(size, keep_first):
 
 
 def short_convolution(u, w):
-    """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the start."""
+    """u [T, C], w [C, taps]: row t = sum over i < taps of w[:, taps - 1 - i] u[t - i], nothing ahead of row 0."""
     taps = w.shape[1]
     out = np.zeros_like(u)
     for t in range(u.shape[0]):
@@ -135,7 +135,7 @@ def decay_of(z):
 
 
 def time_mix_scan(r, k, v, w, u):
-    """r, k, w [T, d], v [T, dv], u [d] of one head: o_t = (S + diag(u) k v^T)^T r, then S <- diag(w) S + k v^T.  Returns o and the last S [d, dv]."""
+    """r, k, w [T, d], v [T, dv], u [d] of one head: o = S^T r + (r . (u k)) v, then row c of S times w_c, plus k_c v.  Returns o and the last S [d, dv]."""
     S = np.zeros((r.shape[1], v.shape[1]))
     out = np.zeros_like(v)
     for t in range(r.shape[0]):
@@ -172,7 +172,7 @@ def feed_forward(h, W, pre, limit):
 
 
 def forward(cfg, W, tokens, taps_out=None):
-    """tokens of ONE sequence -> logits [T, vocab] (float64).  taps_out: a list that receives the residual stream after every layer."""
+    """tokens of ONE sequence -> logits [T, vocab] (float64).  taps_out: a list to which every layer appends the stream it leaves."""
     eps = float(cfg["norm"]["eps"])
     x = norm_around_zero(W["embed"][np.asarray(tokens)], W["embed.norm"], eps)
     for i, L in enumerate(cfg["layers"]):
